@@ -17,7 +17,8 @@ from typing import Optional, Tuple
 
 @dataclass(frozen=True)
 class NormSpec:
-    """A normalisation over the last axis of ``dim`` elements."""
+    """A normalisation over the last axis of ``dim`` elements (``kind``: "rmsnorm", "scalar_rmsnorm", or
+    "layernorm": deviations from the mean over their root mean square, times a weight, no bias)."""
 
     kind: str
     dim: int
@@ -158,18 +159,24 @@ class SinkAttentionSpec:
 class LatentAttentionSpec:
     """Softmax attention whose keys and values are made from one small latent per token, the only
     thing cached: ``c = norm(W_dkv h)`` (``kv_rank`` numbers), per head ``k = W_uk c``,
-    ``v = W_uv c``; queries through a latent of their own, ``q = W_uq norm(W_dq h)``; no
-    positions; ``score = scale * q.k`` over a sliding ``window`` (None: every earlier key), a
-    ``chunk`` (as in :class:`AttentionSpec`) or everything before; with ``gate`` every head's
-    output is multiplied by ``sigmoid(W_g h)`` of that head before the output projection.  The
+    ``v = W_uv c``; queries through a latent of their own, ``q = W_uq norm(W_dq h)``, or with
+    ``q_rank`` None straight from ``h``; ``score = scale * q.k`` over a sliding ``window`` (None: every
+    earlier key), a ``chunk`` (as in :class:`AttentionSpec`) or everything before; with ``gate`` the
+    output is multiplied by ``sigmoid(W_g h)`` before the output projection, head by head
+    (``gate_over="head"``) or element by element of the concatenated heads (``"element"``).  The
     latents' norms divide by the root mean square (``norm_eps`` inside the root) and multiply by a
-    weight."""
+    weight.
+
+    ``rot_dim``: besides its ``head_dim`` elements every head of q has so many that ``position`` rotates,
+    and ``W_dkv h`` has so many rows more, not normed, which after the same rotation are one key part
+    shared by all heads, cached behind the latent; the two parts' products are added before ``scale``
+    (with ``q_rank`` None only).  ``sink``: as in :class:`AttentionSpec`."""
 
     hidden_size: int
     n_heads: int
     head_dim: int
     v_head_dim: int
-    q_rank: int
+    q_rank: Optional[int]
     kv_rank: int
     scale: float
     norm_eps: float
@@ -177,6 +184,36 @@ class LatentAttentionSpec:
     chunk: Optional[int] = None
     gate: bool = True
     kind: str = "latent_attention"
+    gate_over: str = "head"
+    rot_dim: int = 0
+    position: Optional[PositionSpec] = None
+    sink: bool = False
+
+    @property
+    def gate_size(self) -> int:
+        """Rows of the gate's projection."""
+        if not self.gate:
+            return 0
+        return self.n_heads if self.gate_over == "head" else self.n_heads * self.v_head_dim
+
+
+@dataclass(frozen=True)
+class GatedLinearAttentionSpec:
+    """Linear attention with a learned, input-dependent decay per key channel: per request and head a
+    float32 state ``S`` of ``head_dim x v_head_dim``, ``S_t = diag(alpha_t) S_(t-1) + k_t v_t^T``,
+    ``o_t = S_t^T q_t`` (the decay acts on the rows, which belong to key channels); ``q = W_q h *
+    head_dim ** -0.5``, ``alpha = sigmoid(W_a2 (W_a1 h) + b) ** (1 / tau)`` with ``decay_rank`` numbers
+    between the two maps; every head's ``o`` is divided by its root mean square (``norm_eps`` inside the
+    root), times a weight shared by the heads, times ``silu(W_g h)``; then the output projection."""
+
+    hidden_size: int
+    n_heads: int
+    head_dim: int
+    v_head_dim: int
+    decay_rank: int
+    tau: float
+    norm_eps: float
+    kind: str = "gated_linear_attention"
 
 
 @dataclass(frozen=True)
@@ -340,6 +377,16 @@ class GatedFeedForwardSpec:
 
 
 @dataclass(frozen=True)
+class PlainFeedForwardSpec:
+    """``down(act(up(x)))``; ``activation="relu2"``: ``max(z, 0)^2``."""
+
+    hidden_size: int
+    intermediate_size: int
+    activation: str = "relu2"
+    kind: str = "plain_mlp"
+
+
+@dataclass(frozen=True)
 class LayerSpec:
     """One residual block: which mixer, which feed-forward, which norms, how arranged.
 
@@ -353,6 +400,11 @@ class LayerSpec:
     by a learned vector before it is added; ``depth_mix = (index, total)`` makes the layer's result
     stream ``index`` of ``total`` (stream 0: the embedded tokens) and hands on, instead of it, a learned
     mix ``sum_{j <= index} c[j] * stream_j`` of all streams so far.
+
+    ``arrangement="hyper_connections"``: the residual stream is kept in ``streams`` copies ``x_1 .. x_s``
+    (:attr:`ModelSpec.streams`), and every sublayer (mixer or feed-forward) has learned coefficients:
+    ``y = sublayer(norm(sum_s read[s] x_s))``, then, all copies at once, ``x_t <- sum_s mix[s, t] x_s +
+    write[t] y``.
     """
 
     mixer: object
@@ -365,6 +417,7 @@ class LayerSpec:
     input_conv: Optional[object] = None
     sublayer_scale: bool = False
     depth_mix: Optional[Tuple[int, int]] = None
+    streams: int = 1
 
     @property
     def kind(self) -> str:
@@ -404,6 +457,9 @@ class ModelSpec:
     # cap, a scale, ...), as specs with a ``kind``; the Qwen3 decoder has neither.
     stream_parts: Tuple[object, ...] = ()
     logit_parts: Tuple[object, ...] = ()
+    # copies of the residual stream that the layers work on (all equal to the embedded tokens at first;
+    # the final norm reads their sum)
+    streams: int = 1
     extra: dict = field(default_factory=dict, compare=False, hash=False)
 
     def resolved_schedule(self) -> Tuple[Tuple[int, int, bool], ...]:

@@ -1,5 +1,5 @@
 // Paged causal grouped-query attention, the exact and general form: any element type,
-// any head size up to 512 (multiples of 8 with 16-byte loads), any number of heads and groups,
+// any head size up to 1024, values up to 512 (multiples of 8 with 16-byte loads), any number of heads and groups,
 // any page size, optional sliding window or chunks (first_visible in common.h).  One wavefront owns one (token, query head):
 // it walks that token's visible keys 64 at a time (one key per lane), keeps a running
 // maximum and sum in float, and accumulates the weighted values with one lane per
@@ -60,7 +60,7 @@ __global__ void paged_attention_kernel(T* __restrict__ out, const T* __restrict_
                                        int page_size, int window, float scale, int v_dim, long long q_stride,
                                        const float* __restrict__ rel, const int* __restrict__ bucket,
                                        int bucket_len, int sink, int v_transposed, float softcap,
-                                       const float* __restrict__ sink_logit) {
+                                       const float* __restrict__ sink_logit, int v_row) {
   extern __shared__ float lds[];
   const int lane = threadIdx.x & (PYLON_WAVE - 1);
   const int wave = threadIdx.x / PYLON_WAVE;
@@ -125,7 +125,7 @@ __global__ void paged_attention_kernel(T* __restrict__ out, const T* __restrict_
       const T* vr = v_transposed
                         ? v_cache + (static_cast<size_t>(physk / page_size) * n_kv_heads + kvh) * v_dim * page_size +
                               physk % page_size
-                        : v_cache + (static_cast<size_t>(physk) * n_kv_heads + kvh) * v_dim;
+                        : v_cache + (static_cast<size_t>(physk) * n_kv_heads + kvh) * v_row;
       const size_t vstep = v_transposed ? page_size : 1;
 #pragma unroll
       for (int i = 0; i < DIMS_PER_LANE; ++i) {
@@ -162,7 +162,7 @@ static int launch_paged_attention(T* out, const T* q, const T* k_cache, const T*
                                   int head_dim, int page_size, int window, float scale, int v_dim,
                                   long long q_stride, const float* rel, const int* bucket, int bucket_len,
                                   int sink, int v_transposed, float softcap, const float* sink_logit,
-                                  hipStream_t stream) {
+                                  int v_row, hipStream_t stream) {
   const long long items = static_cast<long long>(tokens) * n_heads;
   const long long blocks = (items + ATT_WAVES - 1) / ATT_WAVES;
   dim3 grid((unsigned)blocks), block(ATT_WAVES * PYLON_WAVE);
@@ -171,7 +171,7 @@ static int launch_paged_attention(T* out, const T* q, const T* k_cache, const T*
   hipLaunchKernelGGL((paged_attention_kernel<T, DPL>), grid, block, lds, stream, out, q, k_cache,    \
                      v_cache, block_table, table_width, tok_row, positions, items, n_heads,          \
                      n_kv_heads, head_dim, page_size, window, scale, v_dim, q_stride, rel, bucket,   \
-                     bucket_len, sink, v_transposed, softcap, sink_logit)
+                     bucket_len, sink, v_transposed, softcap, sink_logit, v_row)
   if (v_dim <= 64)
     LAUNCH(1);
   else if (v_dim <= 128)
@@ -186,6 +186,8 @@ static int launch_paged_attention(T* out, const T* q, const T* k_cache, const T*
 
 // q: [tokens, n_heads, head_dim], rows q_stride elements apart; out: [tokens, n_heads, v_dim].
 // Caches: keys [pages*page_size, n_kv_heads, head_dim], values [pages*page_size, n_kv_heads, v_dim].
+// v_row: elements from one value row to the next (v_dim, or more where the values are the first
+// v_dim elements of wider rows: of the keys themselves, say, with v_cache the keys' cache).
 // With v_transposed the values lie as [pages, n_kv_heads, v_dim, page_size].
 // rel: null, or float [rows, n_heads] with bucket: int [bucket_len], every entry a row of rel; or,
 // with bucket null, float [2, n_heads]: per head the factor and the slope of a logarithmic bias.
@@ -199,15 +201,16 @@ extern "C" int pylon_paged_attention(void* out, const void* q, const void* k_cac
                                      int n_kv_heads, int head_dim, int page_size, int window,
                                      float scale, int v_dim, long long q_stride, const float* rel,
                                      const int* bucket, int bucket_len, int sink, int v_transposed,
-                                     float softcap, const float* sink_logit, hipStream_t stream) {
+                                     float softcap, const float* sink_logit, int v_row, hipStream_t stream) {
   PYLON_REQUIRE(pylon_valid_dtype(dtype), "paged_attention: unknown dtype");
   PYLON_REQUIRE(tokens >= 0 && n_heads > 0 && n_kv_heads > 0 && n_heads % n_kv_heads == 0,
                 "paged_attention: %d query heads cannot be grouped over %d key/value heads", n_heads,
                 n_kv_heads);
-  PYLON_REQUIRE(head_dim >= 1 && head_dim <= 512, "paged_attention: head_dim %d must be between 1 and 512", head_dim);
+  PYLON_REQUIRE(head_dim >= 1 && head_dim <= 1024, "paged_attention: head_dim %d must be between 1 and 1024", head_dim);
   PYLON_REQUIRE(page_size > 0 && table_width > 0, "paged_attention: bad page size or table width");
   PYLON_REQUIRE(v_dim >= 1 && v_dim <= 512, "paged_attention: values of 1 to 512 elements, got %d", v_dim);
   PYLON_REQUIRE(q_stride >= static_cast<long long>(n_heads) * head_dim, "paged_attention: q rows overlap");
+  PYLON_REQUIRE(v_row >= v_dim && (v_row == v_dim || !v_transposed), "paged_attention: rows of values overlap, or are transposed and apart");
   PYLON_REQUIRE(rel == nullptr || bucket == nullptr || bucket_len >= 1,
                 "paged_attention: a table of buckets holds at least one entry");
   if (tokens == 0) return 0;
@@ -218,12 +221,12 @@ extern "C" int pylon_paged_attention(void* out, const void* q, const void* k_cac
                                   (const float*)v_cache, block_table, table_width, tok_row, positions,
                                   tokens, n_heads, n_kv_heads, head_dim, page_size, window, scale, v_dim,
                                   q_stride, rel, bucket, bucket_len, sink, v_transposed, softcap, sink_logit,
-                                  stream);
+                                  v_row, stream);
   else
     launch_paged_attention<bf16_t>((bf16_t*)out, (const bf16_t*)q, (const bf16_t*)k_cache,
                                    (const bf16_t*)v_cache, block_table, table_width, tok_row, positions,
                                    tokens, n_heads, n_kv_heads, head_dim, page_size, window, scale, v_dim,
                                    q_stride, rel, bucket, bucket_len, sink, v_transposed, softcap, sink_logit,
-                                  stream);
+                                  v_row, stream);
   PYLON_LAUNCHED("paged_attention");
 }

@@ -10,7 +10,7 @@
 template <typename T>
 __global__ void embed_kernel(float* __restrict__ out, const T* __restrict__ table,
                              const int* __restrict__ ids, const int* __restrict__ chosen, int hidden,
-                             int vocab, float scale) {
+                             int vocab, float scale, int copies) {
   const int t = blockIdx.x;
   int id = ids[t];
   if (id < 0 && chosen != nullptr) id = chosen[-1 - id];
@@ -18,25 +18,30 @@ __global__ void embed_kernel(float* __restrict__ out, const T* __restrict__ tabl
   id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
   const T* row = table + static_cast<size_t>(id) * hidden;
   float* dst = out + static_cast<size_t>(t) * hidden;
-  for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_float(row[i]) * scale;
+  const size_t apart = static_cast<size_t>(gridDim.x) * hidden;  // from one copy to the next
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+    const float v = to_float(row[i]) * scale;
+    for (int c = 0; c < copies; ++c) dst[c * apart + i] = v;
+  }
 }
 
 // chosen may be null; then every id must be a table row.  The host guarantees that a
-// negative id -(1 + s) names an entry s inside chosen.
+// negative id -(1 + s) names an entry s inside chosen.  out: [copies, tokens, hidden], all copies equal.
 extern "C" int pylon_embed(float* out, const void* table, int table_dtype, const int* ids,
-                           const int* chosen, int tokens, int hidden, int vocab, float scale,
+                           const int* chosen, int tokens, int hidden, int vocab, float scale, int copies,
                            hipStream_t stream) {
   PYLON_REQUIRE(pylon_valid_dtype(table_dtype), "embed: unknown table dtype %d", table_dtype);
   PYLON_REQUIRE(tokens >= 0 && hidden > 0 && vocab > 0, "embed: bad sizes tokens=%d hidden=%d vocab=%d",
                 tokens, hidden, vocab);
+  PYLON_REQUIRE(copies >= 1, "embed: at least one copy");
   if (tokens == 0) return 0;
   dim3 grid(tokens), block(256);
   if (table_dtype == PYLON_F32)
     hipLaunchKernelGGL(embed_kernel<float>, grid, block, 0, stream, out, (const float*)table, ids,
-                       chosen, hidden, vocab, scale);
+                       chosen, hidden, vocab, scale, copies);
   else
     hipLaunchKernelGGL(embed_kernel<bf16_t>, grid, block, 0, stream, out, (const bf16_t*)table, ids,
-                       chosen, hidden, vocab, scale);
+                       chosen, hidden, vocab, scale, copies);
   PYLON_LAUNCHED("embed");
 }
 
@@ -495,6 +500,56 @@ extern "C" int pylon_gated_act(void* out, int out_dtype, const void* gate_up, in
   else GO(bf16_t, bf16_t);
 #undef GO
   PYLON_LAUNCHED("gated_act");
+}
+
+// ---- the square of relu: out = max(x, 0)^2 -----------------------------------------------------
+template <typename TI, typename TO>
+__global__ void relu2_kernel(TO* __restrict__ out, const TI* __restrict__ x, size_t total) {
+  size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
+  const size_t step = static_cast<size_t>(gridDim.x) * blockDim.x;
+  for (; i < total; i += step) {
+    const float v = fmaxf(to_float(x[i]), 0.f);
+    out[i] = from_float<TO>(v * v);
+  }
+}
+
+// Eight elements (16 bytes of bfloat16) a thread.
+__global__ void relu2_bf16x8_kernel(uint4* __restrict__ out, const uint4* __restrict__ x, size_t total) {
+  size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
+  const size_t step = static_cast<size_t>(gridDim.x) * blockDim.x;
+  for (; i < total; i += step) {
+    const uint4 raw = x[i];
+    const uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
+    uint32_t r[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float a = fmaxf(__uint_as_float(w[j] << 16), 0.f), b = fmaxf(__uint_as_float(w[j] & 0xffff0000u), 0.f);
+      r[j] = static_cast<uint32_t>(float_to_bf16_bits(a * a)) | (static_cast<uint32_t>(float_to_bf16_bits(b * b)) << 16);
+    }
+    out[i] = uint4{r[0], r[1], r[2], r[3]};
+  }
+}
+
+// x and out may be the same tensor where their types are.
+extern "C" int pylon_relu2(void* out, int out_dtype, const void* x, int in_dtype, long long count, hipStream_t stream) {
+  PYLON_REQUIRE(pylon_valid_dtype(in_dtype) && pylon_valid_dtype(out_dtype) && count >= 0, "relu2: bad arguments");
+  if (count == 0) return 0;
+  const bool wide = in_dtype == PYLON_BF16 && out_dtype == PYLON_BF16 && count % 8 == 0 &&
+                    ((reinterpret_cast<uintptr_t>(out) | reinterpret_cast<uintptr_t>(x)) & 15) == 0;
+  const size_t total = wide ? static_cast<size_t>(count) / 8 : static_cast<size_t>(count);
+  size_t blocks = (total + 255) / 256;
+  if (blocks > 65535u * 16u) blocks = 65535u * 16u;
+  dim3 grid((unsigned)blocks), block(256);
+  if (wide) hipLaunchKernelGGL(relu2_bf16x8_kernel, grid, block, 0, stream, (uint4*)out, (const uint4*)x, total);
+  else if (in_dtype == PYLON_F32 && out_dtype == PYLON_F32)
+    hipLaunchKernelGGL((relu2_kernel<float, float>), grid, block, 0, stream, (float*)out, (const float*)x, total);
+  else if (in_dtype == PYLON_F32)
+    hipLaunchKernelGGL((relu2_kernel<float, bf16_t>), grid, block, 0, stream, (bf16_t*)out, (const float*)x, total);
+  else if (out_dtype == PYLON_F32)
+    hipLaunchKernelGGL((relu2_kernel<bf16_t, float>), grid, block, 0, stream, (float*)out, (const bf16_t*)x, total);
+  else
+    hipLaunchKernelGGL((relu2_kernel<bf16_t, bf16_t>), grid, block, 0, stream, (bf16_t*)out, (const bf16_t*)x, total);
+  PYLON_LAUNCHED("relu2");
 }
 
 // ---- scaling in place ------------------------------------------------------------------------

@@ -10,7 +10,15 @@
 // head_project: out[t, h, :] = gate[t, h] * x[t, h, :] @ m[h] with m [heads, n_in, n_out]; a
 //   workgroup keeps the inputs of a few tokens in LDS and walks 64 columns of m[h] once for all of
 //   them, its four waves a quarter of n_in each; sums in float in one fixed order, whatever the batch.
+//   The heads of x and of out may lie apart (parts of wider heads), and the gate may come as raw logits
+//   of x's type, one per head or per element, whose sigmoid is taken here.
 // gate_heads: x[t, h, :] *= gate[t, h] in place.
+//
+// Where a part of every key carries positions, the row of a token in the cache is [c | r]: the normed
+// latent and one rotated key part r that all heads share; a query in that space is [q' | rotated part of
+// q], so that the score is still one product of the two and the values are still the latent's elements.
+// latent_rotate: from the projection's rows, c normed and r rotated into the token's cache slot, and the
+//   rotated part of every head of q into the places it has in the query rows.
 #include "common.h"
 
 #define LP_THREADS 256
@@ -65,6 +73,104 @@ extern "C" int pylon_latent_prepare(void* q_latent, void* c_cache, float* gate_o
   PYLON_LAUNCHED("latent_prepare");
 }
 
+template <typename T>
+__global__ void __launch_bounds__(LP_THREADS)
+latent_rotate_kernel(T* __restrict__ q_out, T* __restrict__ cache, const T* __restrict__ proj, long long ld, int q_off,
+                     int heads, int dim, int rot, int c_off, int rank, const float* __restrict__ c_weight, float eps,
+                     const float* __restrict__ inv_freq, float rot_scale, int interleaved,
+                     const int* __restrict__ positions, const int* __restrict__ slot_map, int store) {
+  extern __shared__ float turn[];  // [2][rot / 2]: cosines and sines of the token's angles, times rot_scale
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const T* row = proj + static_cast<size_t>(t) * ld;
+  const int half = rot / 2, width = rank + rot;
+  if (inv_freq != nullptr) {
+    const float pos = static_cast<float>(positions[t]);
+    for (int i = tid; i < half; i += LP_THREADS) {
+      float sn, cs;
+      sincosf(pos * inv_freq[i], &sn, &cs);
+      turn[i] = cs * rot_scale;
+      turn[half + i] = sn * rot_scale;
+    }
+  }
+  __syncthreads();
+  // pair i of a part: neighbours (2i, 2i + 1), or halves (i, i + rot / 2)
+  auto rotate = [&](const T* src, T* dst, int i) {
+    const int a = interleaved ? 2 * i : i, b = interleaved ? 2 * i + 1 : i + half;
+    const float u = to_float(src[a]), v = to_float(src[b]);
+    float x = u, y = v;
+    if (inv_freq != nullptr) {
+      const float cs = turn[i], sn = turn[half + i];
+      x = u * cs - v * sn;
+      y = v * cs + u * sn;
+    }
+    dst[a] = from_float<T>(x);
+    dst[b] = from_float<T>(y);
+  };
+  for (int e = tid; e < heads * half; e += LP_THREADS) {
+    const int h = e / half, i = e - h * half;
+    rotate(row + q_off + static_cast<size_t>(h) * (dim + rot) + dim,
+           q_out + (static_cast<size_t>(t) * heads + h) * width + rank, i);
+  }
+  if (!store) return;
+  const T* c = row + c_off;
+  float sq = 0.f;
+  for (int i = tid; i < rank; i += LP_THREADS) {
+    const float v = to_float(c[i]);
+    sq = fmaf(v, v, sq);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(sq, scratch) / static_cast<float>(rank) + eps);
+  T* dst = cache + static_cast<size_t>(slot_map[t]) * width;
+  for (int i = tid; i < rank; i += LP_THREADS) dst[i] = from_float<T>(to_float(c[i]) * inv * c_weight[i]);
+  for (int i = tid; i < half; i += LP_THREADS) rotate(c + rank, dst + rank, i);
+}
+
+// proj: [tokens, ld] of dtype holding, from q_off, the heads of q as [dim | rot] each, and from c_off the
+// latent (rank elements) and behind it the shared rotated key part (rot elements).  q_out: [tokens, heads,
+// rank + rot], of which only the last rot elements of every head are written.  cache: [slots, rank + rot].
+// inv_freq: float [rot / 2], or null (the parts are copied as they are); rot_scale multiplies every cosine
+// and sine.
+extern "C" int pylon_latent_rotate(void* q_out, void* cache, const void* proj, int dtype, long long ld, int q_off,
+                                   int heads, int dim, int rot, int c_off, int rank, const float* c_weight, float eps,
+                                   const float* inv_freq, float rot_scale, int interleaved, const int* positions,
+                                   const int* slot_map, int tokens, int store, hipStream_t stream) {
+  PYLON_REQUIRE(pylon_valid_dtype(dtype), "latent_rotate: unknown dtype");
+  PYLON_REQUIRE(tokens >= 0 && heads > 0 && dim > 0 && rot >= 0 && rot % 2 == 0 && rot <= 1024 && rank > 0,
+                "latent_rotate: bad sizes");
+  PYLON_REQUIRE(q_off >= 0 && c_off >= 0 && q_off + static_cast<long long>(heads) * (dim + rot) <= ld &&
+                    c_off + static_cast<long long>(rank) + rot <= ld,
+                "latent_rotate: q or the latent lie outside the projection's rows");
+  PYLON_REQUIRE(inv_freq == nullptr || positions != nullptr, "latent_rotate: a rotation needs positions");
+  PYLON_REQUIRE(!store || (cache != nullptr && slot_map != nullptr && c_weight != nullptr),
+                "latent_rotate: storing needs cache, slots and the norm's weight");
+  if (tokens == 0) return 0;
+  const size_t lds = sizeof(float) * (rot > 0 ? rot : 2);
+  if (dtype == PYLON_F32)
+    hipLaunchKernelGGL((latent_rotate_kernel<float>), dim3(tokens), dim3(LP_THREADS), lds, stream, (float*)q_out,
+                       (float*)cache, (const float*)proj, ld, q_off, heads, dim, rot, c_off, rank, c_weight, eps,
+                       inv_freq, rot_scale, interleaved, positions, slot_map, store);
+  else
+    hipLaunchKernelGGL((latent_rotate_kernel<bf16_t>), dim3(tokens), dim3(LP_THREADS), lds, stream, (bf16_t*)q_out,
+                       (bf16_t*)cache, (const bf16_t*)proj, ld, q_off, heads, dim, rot, c_off, rank, c_weight, eps,
+                       inv_freq, rot_scale, interleaved, positions, slot_map, store);
+  PYLON_LAUNCHED("latent_rotate");
+}
+
+// What multiplies an output of the per-head product: a float gate per (token, head), or the sigmoid of
+// raw logits (per: outputs that share one, a head's or 1).
+template <typename TX>
+struct HeadGate {
+  const float* heads;
+  const TX* logits;
+  long long logit_stride;
+  int per;
+  __device__ __forceinline__ float at(int t, int n_heads, int h, int n_out, int o) const {
+    if (logits != nullptr)
+      return 1.0f / (1.0f + expf(-to_float(logits[static_cast<size_t>(t) * logit_stride + (h * n_out + o) / per])));
+    return heads != nullptr ? heads[static_cast<size_t>(t) * n_heads + h] : 1.f;
+  }
+};
+
 #define HP_THREADS 256
 #define HP_TOKENS 8
 #define HP_COLS 64   // outputs of a workgroup
@@ -72,14 +178,15 @@ extern "C" int pylon_latent_prepare(void* q_latent, void* c_cache, float* gate_o
 
 template <typename TX, typename TM>
 __global__ void __launch_bounds__(HP_THREADS)
-head_project_kernel(TX* __restrict__ out, const TX* __restrict__ x, long long x_stride, const TM* __restrict__ m,
-                    const float* __restrict__ gate, int tokens, int heads, int n_in, int n_out) {
+head_project_kernel(TX* __restrict__ out, long long out_stride, int out_hstride, const TX* __restrict__ x,
+                    long long x_stride, int x_hstride, const TM* __restrict__ m, HeadGate<TX> gate, int tokens,
+                    int heads, int n_in, int n_out) {
   extern __shared__ float xs[];  // [HP_TOKENS, n_in], then the slices' partial sums [HP_SLICES, HP_TOKENS, HP_COLS]
   float* partial = xs + HP_TOKENS * n_in;
   const int t0 = blockIdx.x * HP_TOKENS, h = blockIdx.y, tid = threadIdx.x;
   for (int i = tid; i < HP_TOKENS * n_in; i += HP_THREADS) {
     const int tt = i / n_in, k = i - tt * n_in;
-    xs[i] = (t0 + tt < tokens) ? to_float(x[static_cast<size_t>(t0 + tt) * x_stride + static_cast<size_t>(h) * n_in + k])
+    xs[i] = (t0 + tt < tokens) ? to_float(x[static_cast<size_t>(t0 + tt) * x_stride + static_cast<size_t>(h) * x_hstride + k])
                                : 0.f;
   }
   __syncthreads();
@@ -110,8 +217,8 @@ head_project_kernel(TX* __restrict__ out, const TX* __restrict__ x, long long x_
     float sum = partial[tt * HP_COLS + c];
 #pragma unroll
     for (int sl = 1; sl < HP_SLICES; ++sl) sum += partial[(sl * HP_TOKENS + tt) * HP_COLS + c];
-    const float g = gate != nullptr ? gate[static_cast<size_t>(t0 + tt) * heads + h] : 1.f;
-    out[(static_cast<size_t>(t0 + tt) * heads + h) * n_out + oc] = from_float<TX>(sum * g);
+    const float g = gate.at(t0 + tt, heads, h, n_out, oc);
+    out[static_cast<size_t>(t0 + tt) * out_stride + static_cast<size_t>(h) * out_hstride + oc] = from_float<TX>(sum * g);
   }
 }
 
@@ -122,15 +229,15 @@ head_project_kernel(TX* __restrict__ out, const TX* __restrict__ x, long long x_
 #define HW_COLS 128
 
 __global__ void __launch_bounds__(HP_THREADS)
-head_project_wide_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ x, long long x_stride,
-                         const bf16_t* __restrict__ m, const float* __restrict__ gate, int tokens, int heads, int n_in,
-                         int n_out) {
+head_project_wide_kernel(bf16_t* __restrict__ out, long long out_stride, int out_hstride, const bf16_t* __restrict__ x,
+                         long long x_stride, int x_hstride, const bf16_t* __restrict__ m, HeadGate<bf16_t> gate,
+                         int tokens, int heads, int n_in, int n_out) {
   extern __shared__ float xs[];  // [HP_TOKENS, n_in], then the waves' partial sums [4, HP_TOKENS, HW_COLS]
   float* partial = xs + HP_TOKENS * n_in;
   const int t0 = blockIdx.x * HP_TOKENS, h = blockIdx.y, c0 = blockIdx.z * HW_COLS, tid = threadIdx.x;
   for (int i = tid; i < HP_TOKENS * n_in; i += HP_THREADS) {
     const int tt = i / n_in, k = i - tt * n_in;
-    xs[i] = (t0 + tt < tokens) ? to_float(x[static_cast<size_t>(t0 + tt) * x_stride + static_cast<size_t>(h) * n_in + k])
+    xs[i] = (t0 + tt < tokens) ? to_float(x[static_cast<size_t>(t0 + tt) * x_stride + static_cast<size_t>(h) * x_hstride + k])
                                : 0.f;
   }
   __syncthreads();
@@ -178,20 +285,30 @@ head_project_wide_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ x,
     float sum = partial[tt * HW_COLS + c];
 #pragma unroll
     for (int wv = 1; wv < 4; ++wv) sum += partial[(wv * HP_TOKENS + tt) * HW_COLS + c];
-    const float g = gate != nullptr ? gate[static_cast<size_t>(t0 + tt) * heads + h] : 1.f;
-    out[(static_cast<size_t>(t0 + tt) * heads + h) * n_out + c0 + c] = from_float<bf16_t>(sum * g);
+    const float g = gate.at(t0 + tt, heads, h, n_out, c0 + c);
+    out[static_cast<size_t>(t0 + tt) * out_stride + static_cast<size_t>(h) * out_hstride + c0 + c] = from_float<bf16_t>(sum * g);
   }
 }
 
-// x: [tokens, heads, n_in], rows x_stride elements apart; m: [heads, n_in, n_out]; gate: null or
-// float [tokens, heads]; out: [tokens, heads, n_out] of x's type.  m may be float while x is bfloat16.
-extern "C" int pylon_head_project(void* out, const void* x, int x_dtype, long long x_stride, const void* m,
-                                  int m_dtype, const float* gate, int tokens, int heads, int n_in, int n_out,
-                                  hipStream_t stream) {
+// x: [tokens, heads, n_in], rows x_stride and heads x_hstride elements apart; m: [heads, n_in, n_out]; gate:
+// null or float [tokens, heads]; gate_logits: null (and then at most one of the two) or, of x's type, [tokens,
+// heads * n_out / gate_per], rows gate_stride apart; out: [tokens, heads, n_out] of x's type, rows out_stride
+// and heads out_hstride apart.  m may be float while x is bfloat16.
+extern "C" int pylon_head_project(void* out, long long out_stride, int out_hstride, const void* x, int x_dtype,
+                                  long long x_stride, int x_hstride, const void* m, int m_dtype, const float* gate,
+                                  const void* gate_logits, long long gate_stride, int gate_per, int tokens, int heads,
+                                  int n_in, int n_out, hipStream_t stream) {
   PYLON_REQUIRE(pylon_valid_dtype(x_dtype) && pylon_valid_dtype(m_dtype), "head_project: unknown dtype");
   PYLON_REQUIRE(tokens >= 0 && heads > 0 && n_in > 0 && n_out > 0, "head_project: sizes must be positive");
   PYLON_REQUIRE(heads <= 65535, "head_project: too many heads for one launch");
-  PYLON_REQUIRE(x_stride >= static_cast<long long>(heads) * n_in, "head_project: rows of x overlap");
+  PYLON_REQUIRE(x_hstride >= n_in && x_stride >= static_cast<long long>(heads - 1) * x_hstride + n_in,
+                "head_project: rows of x overlap");
+  PYLON_REQUIRE(out_hstride >= n_out && out_stride >= static_cast<long long>(heads - 1) * out_hstride + n_out,
+                "head_project: rows of the result overlap");
+  PYLON_REQUIRE(gate == nullptr || gate_logits == nullptr, "head_project: gates or their logits, not both");
+  PYLON_REQUIRE(gate_logits == nullptr || (gate_per >= 1 && (static_cast<long long>(heads) * n_out) % gate_per == 0 &&
+                                           gate_stride >= static_cast<long long>(heads) * n_out / gate_per),
+                "head_project: the gates' logits do not match the outputs");
   const size_t lds = sizeof(float) * (HP_TOKENS * n_in + HP_SLICES * HP_TOKENS * HP_COLS);
   PYLON_REQUIRE(lds <= 64 * 1024, "head_project: %d inputs per head do not fit LDS", n_in);
   PYLON_REQUIRE(!(x_dtype == PYLON_F32 && m_dtype == PYLON_BF16), "head_project: float inputs take a float matrix");
@@ -201,8 +318,10 @@ extern "C" int pylon_head_project(void* out, const void* x, int x_dtype, long lo
     const int zw = (n_out + HW_COLS - 1) / HW_COLS;
     if (wide_lds <= 64 * 1024 && zw <= 65535) {
       hipLaunchKernelGGL(head_project_wide_kernel, dim3((tokens + HP_TOKENS - 1) / HP_TOKENS, heads, zw),
-                         dim3(HP_THREADS), wide_lds, stream, (bf16_t*)out, (const bf16_t*)x, x_stride,
-                         (const bf16_t*)m, gate, tokens, heads, n_in, n_out);
+                         dim3(HP_THREADS), wide_lds, stream, (bf16_t*)out, out_stride, out_hstride, (const bf16_t*)x,
+                         x_stride, x_hstride, (const bf16_t*)m,
+                         (HeadGate<bf16_t>{gate, (const bf16_t*)gate_logits, gate_stride, gate_per}), tokens, heads, n_in,
+                         n_out);
       PYLON_LAUNCHED("head_project");
     }
   }
@@ -210,8 +329,9 @@ extern "C" int pylon_head_project(void* out, const void* x, int x_dtype, long lo
   PYLON_REQUIRE(zs <= 65535, "head_project: too many outputs per head for one launch");
   dim3 grid((tokens + HP_TOKENS - 1) / HP_TOKENS, heads, zs), block(HP_THREADS);
 #define GO(TX, TM)                                                                                              \
-  hipLaunchKernelGGL((head_project_kernel<TX, TM>), grid, block, lds, stream, (TX*)out, (const TX*)x, x_stride, \
-                     (const TM*)m, gate, tokens, heads, n_in, n_out)
+  hipLaunchKernelGGL((head_project_kernel<TX, TM>), grid, block, lds, stream, (TX*)out, out_stride, out_hstride, \
+                     (const TX*)x, x_stride, x_hstride, (const TM*)m,                                           \
+                     (HeadGate<TX>{gate, (const TX*)gate_logits, gate_stride, gate_per}), tokens, heads, n_in, n_out)
   if (x_dtype == PYLON_F32) GO(float, float);
   else if (m_dtype == PYLON_F32) GO(bf16_t, float);
   else GO(bf16_t, bf16_t);

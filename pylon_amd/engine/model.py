@@ -10,6 +10,9 @@ tokens), "logits" parts after the head (``forward(logits, ctx) -> logits``, floa
 per wanted token; under graph replay they must write in place).  A schedule entry with
 ``add_embedding`` has the embedded tokens (after the stream parts) added to the stream once more
 before its run: how a model that runs a stretch of layers several times feeds every further pass.
+A model may keep the residual stream in several copies (``ModelSpec.streams``), ``[copies, tokens,
+dim]``: they start as the embedded tokens, the layers' arrangement says how they change, and the final
+norm reads their sum.
 """
 from __future__ import annotations
 
@@ -35,6 +38,11 @@ class Model(Part):
         self.device = torch.device(device)
         self.schedule = spec.resolved_schedule()
         self.embedding_again = spec.embedding_again()
+        if spec.streams < 1 or any(layer.streams != spec.streams for layer in spec.layers):
+            raise ValueError(f"the model keeps its residual stream in {spec.streams} copies, its layers in "
+                             f"{sorted({layer.streams for layer in spec.layers})}")
+        if spec.streams > 1 and (spec.stream_parts or any(self.embedding_again)):
+            raise ValueError("parts on the embedded tokens and tokens added again need a residual stream in one copy")
         self.add_param("embed", (spec.vocab_size, spec.hidden_size), dtype, device)
         if not spec.tie_word_embeddings:
             self.add_param("lm_head", (spec.vocab_size, spec.hidden_size), dtype, device)
@@ -97,7 +105,7 @@ class Model(Part):
         """Run the step's tokens through every scheduled layer, from and into the cache.
         Returns float32 logits ``[n_logits, vocab]`` (None when no logits are wanted)."""
         resid = ops.embed(ctx.token_ids, self.params["embed"], scale=self.spec.embedding_scale,
-                          chosen=ctx.chosen)
+                          chosen=ctx.chosen, copies=self.spec.streams)
         for part in self.stream_parts:
             resid = part.forward(resid, ctx)
         # a schedule may add the embedded tokens to the stream again before some of its runs

@@ -56,19 +56,22 @@ def _dev(t: Optional[torch.Tensor], name: str, dtype=None) -> int:
 
 
 def embed(ids: torch.Tensor, table: torch.Tensor, *, scale: float = 1.0,
-          out: Optional[torch.Tensor] = None, chosen: Optional[torch.Tensor] = None) -> torch.Tensor:
+          out: Optional[torch.Tensor] = None, chosen: Optional[torch.Tensor] = None,
+          copies: int = 1) -> torch.Tensor:
     """float32 ``out[t] = table[ids[t]] * scale``.  With ``chosen`` (int32, on the device) an
-    id ``-(1 + s)`` is replaced by ``chosen[s]``: the token a sampler left there."""
+    id ``-(1 + s)`` is replaced by ``chosen[s]``: the token a sampler left there.  ``copies > 1``:
+    the result is ``[copies, tokens, hidden]``, every copy the same."""
     tokens = ids.numel()
     vocab, hidden = table.shape
+    shape = (tokens, hidden) if copies == 1 else (copies, tokens, hidden)
     if out is None:
-        out = torch.empty((tokens, hidden), dtype=torch.float32, device=table.device)
-    elif out.shape != (tokens, hidden):
-        raise KernelError(f"embed: out has shape {tuple(out.shape)}, expected {(tokens, hidden)}")
+        out = torch.empty(shape, dtype=torch.float32, device=table.device)
+    elif out.shape != shape:
+        raise KernelError(f"embed: out has shape {tuple(out.shape)}, expected {shape}")
     _lib.call("pylon_embed", _dev(out, "out", torch.float32), _dev(table, "table"),
               dtype_code(table.dtype), _dev(ids, "ids", torch.int32),
               None if chosen is None else _dev(chosen, "chosen", torch.int32), tokens, hidden, vocab,
-              float(scale), _stream())
+              float(scale), int(copies), _stream())
     return out
 
 
@@ -214,7 +217,8 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                     bucket: Optional[torch.Tensor] = None, sink: bool = False,
                     v_transposed: bool = False, chunk: Optional[int] = None,
                     log_bias: Optional[torch.Tensor] = None, softcap: Optional[float] = None,
-                    sink_logit: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    sink_logit: Optional[torch.Tensor] = None,
+                    values_in_keys: Optional[int] = None) -> torch.Tensor:
     """Causal attention of each token over its request's cached keys ``<=`` its position (with
     ``window`` the last so many, with ``chunk`` those of its own chunk: :func:`mask_code`).
     ``q`` is ``[tokens, heads, head_dim]`` and may be a slice of wider rows (a fused
@@ -224,7 +228,9 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     ``a[head] * log(1 + b[head] * (i - j))`` off it instead; ``sink`` adds one to the softmax's
     denominator.  With ``v_transposed`` the values lie as ``[pages, kv_heads, v_dim, page_size]``.
     ``softcap``: the scaled score ``s`` becomes ``softcap * tanh(s / softcap)``.  ``sink_logit``
-    (float32 ``[heads]``): ``exp(sink_logit[head])`` joins the denominator, unscaled and uncapped."""
+    (float32 ``[heads]``): ``exp(sink_logit[head])`` joins the denominator, unscaled and uncapped.
+    ``values_in_keys = n``: a key's value is the first ``n`` elements of its own row (``v_cache`` is
+    then ``k_cache`` itself)."""
     if q.dim() != 3:
         raise KernelError("paged_attention takes q as [tokens, heads, head_dim]")
     if sink_logit is not None and (sink or sink_logit.shape != (q.shape[1],)):
@@ -239,7 +245,11 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     if k_cache.dim() != 4 or v_cache.dim() != 4 or tuple(k_cache.shape[:3]) != v_shape[:3]:
         raise KernelError("paged_attention: caches must be [pages, page_size, kv_heads, head_dim]")
     pages, psize, n_kv_heads, hd = k_cache.shape
-    v_dim = v_shape[3]
+    v_dim = v_row = v_shape[3]
+    if values_in_keys is not None:
+        if v_cache is not k_cache or v_transposed or not 1 <= values_in_keys <= hd:
+            raise KernelError("paged_attention: values inside the keys are the first elements of the keys' own rows")
+        v_dim = int(values_in_keys)
     if q.stride(2) != 1 or q.stride(1) != head_dim or (tokens > 1 and q.stride(0) < n_heads * head_dim):
         raise KernelError("paged_attention: the heads of a q row must lie side by side")
     if (rel is None) != (bucket is None):
@@ -273,7 +283,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
               page_size, mask_code(window, chunk), float(scale), v_dim, q.stride(0) if tokens > 1 else n_heads * head_dim,
               _dev(rel, "rel", torch.float32), _dev(bucket, "bucket", torch.int32),
               0 if bucket is None else bucket.numel(), 1 if sink else 0, 1 if v_transposed else 0,
-              float(softcap or 0.0), _dev(sink_logit, "sink_logit", torch.float32), _stream())
+              float(softcap or 0.0), _dev(sink_logit, "sink_logit", torch.float32), v_row, _stream())
     return out
 
 
@@ -452,6 +462,48 @@ def depth_mix(resid: torch.Tensor, delta: Optional[torch.Tensor], streams: torch
     return out
 
 
+STREAM_COPIES = 16  # most copies of a residual stream that the norm kernel mixes
+
+
+def stream_norm(resid: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Tensor, eps: float,
+                out_dtype: torch.dtype, *, centre: bool, mix: Optional[torch.Tensor] = None,
+                write: Optional[torch.Tensor] = None, read: Optional[torch.Tensor] = None,
+                row_idx: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """A residual stream in several copies ``resid`` (float32 ``[copies, tokens, dim]``; one copy may
+    come as ``[tokens, dim]``), updated in place by the last sublayer's output ``d`` (``delta``, or the
+    sum of a stack of float32 partial sums), ``x_t <- sum_s mix[s, t] x_s + write[t] d``, and the norm
+    of ``u = sum_t read[t] x_t``: ``(u - mean) / sqrt(var + eps) * weight`` with ``centre`` (layer norm,
+    the variance from the deviations), ``u / sqrt(mean(u^2) + eps) * weight`` without.  ``mix`` None:
+    every copy stays itself; ``write`` and ``read`` None: ones.  With ``row_idx`` only those rows are
+    normed and ``resid`` is left as it is; without ``delta`` nothing is mixed."""
+    if resid.dim() not in (2, 3) or resid.dtype != torch.float32 or not resid.is_contiguous():
+        raise KernelError("stream_norm takes a contiguous float32 [tokens, dim] or [copies, tokens, dim]")
+    copies = resid.shape[0] if resid.dim() == 3 else 1
+    tokens, dim = resid.shape[-2:]
+    if not 1 <= copies <= STREAM_COPIES:
+        raise KernelError(f"stream_norm: 1 to {STREAM_COPIES} copies of the stream, got {copies}")
+    for name, tensor, shape in (("mix", mix, (copies, copies)), ("write", write, (copies,)), ("read", read, (copies,)),
+                                ("weight", weight, (dim,))):
+        if tensor is not None and tensor.shape != shape:
+            raise KernelError(f"stream_norm: {name} must have shape {shape}, got {tuple(tensor.shape)}")
+    n_delta, delta_stride = 1, 0
+    if delta is not None:
+        if delta.dim() == 3:
+            n_delta, delta_stride = delta.shape[0], delta.shape[1] * delta.shape[2]
+            if delta.dtype != torch.float32:
+                raise KernelError("stream_norm: a stack of partial sums is float32")
+        if tuple(delta.shape[-2:]) != (tokens, dim):
+            raise KernelError("stream_norm: delta and resid differ in shape")
+    rows = tokens if row_idx is None else row_idx.numel()
+    out = torch.empty((rows, dim), dtype=out_dtype, device=resid.device)
+    _lib.call("pylon_stream_norm", _dev(out, "out"), dtype_code(out_dtype), _dev(resid, "resid", torch.float32),
+              tokens * dim, copies, _dev(delta, "delta"), dtype_code(delta.dtype) if delta is not None else F32, n_delta,
+              delta_stride, _dev(mix, "mix", torch.float32), _dev(write, "write", torch.float32),
+              _dev(read, "read", torch.float32), _dev(weight, "weight", torch.float32),
+              _dev(row_idx, "row_idx", torch.int32), rows, dim, float(eps), 1 if centre else 0, _stream())
+    return out
+
+
 def token_shift(h: torch.Tensor, shift: torch.Tensor, state: torch.Tensor, row_start: torch.Tensor,
                 row_slots: torch.Tensor, *, rows: int, max_count: int, out_dtype: torch.dtype) -> torch.Tensor:
     """``h[t] + (h[t - 1] - h[t]) * shift`` per channel and request, zeros before a request's first
@@ -588,6 +640,46 @@ def retention_recurrent(proj: torch.Tensor, state: torch.Tensor, decay: torch.Te
               _dev(positions, "positions", torch.int32), _dev(row_start, "row_start", torch.int32),
               _dev(row_slots, "row_slots", torch.int32), rows, heads, dim, vdim, float(eps), float(k_scale),
               _stream())
+    return out
+
+
+def gla_ok(dim: int, vdim: int) -> bool:
+    """Whether :func:`gla_recurrent` has a layout for heads of ``dim x vdim`` (the kernel's own rule)."""
+    if not (1 <= dim <= 1024 and 1 <= vdim <= 1024):
+        return False
+    return -(-dim // min(dim, 1024 // vdim)) <= 64
+
+
+def gla_recurrent(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_bias: torch.Tensor,
+                  norm_weight: torch.Tensor, row_start: torch.Tensor, row_slots: torch.Tensor, *, rows: int, heads: int,
+                  dim: int, vdim: int, rank: int, tau: float, eps: float, q_scale: float) -> torch.Tensor:
+    """Gated linear attention, token by token: ``proj`` ``[tokens, 2 heads dim + 2 heads vdim + rank]``
+    holds q, k, v, the output gate and the decays' low-rank logits side by side; with ``z = a2 low +
+    a2_bias`` (float32 ``[heads * dim, rank]`` and ``[heads * dim]``) a key channel's decay is
+    ``sigmoid(z)^(1/tau)``; ``S <- diag(decay) S + k v^T``, ``o = S^T (q_scale q)``.  ``state`` (float32
+    ``[slots, heads, dim, vdim]``) is read and left up to date.  Returns ``o / rms(o) * norm_weight *
+    silu(gate)`` as ``[tokens, heads * vdim]``."""
+    tokens = proj.shape[0]
+    q, v = heads * dim, heads * vdim
+    if proj.dim() != 2 or proj.shape[1] != 2 * q + 2 * v + rank or proj.stride(1) != 1:
+        raise KernelError("gla: the projection's rows must hold q, k, v, the gate and the decays' logits")
+    if state.dim() != 4 or state.shape[1:] != (heads, dim, vdim):
+        raise KernelError(f"gla: state must be [slots, {heads}, {dim}, {vdim}]")
+    if a2.shape != (q, rank) or a2_bias.shape != (q,) or norm_weight.shape != (vdim,):
+        raise KernelError("gla: a2 must be [heads * dim, rank] with a bias per row, and the norm have vdim weights")
+    if row_start.numel() != rows + 1 or row_slots.numel() != rows:
+        raise KernelError("gla: one start per row and one more, and one slot per row")
+    if not gla_ok(dim, vdim):
+        raise KernelError(f"gla does not take heads of {dim} x {vdim}")
+    if not proj.is_cuda:
+        raise KernelError("proj must live on the GPU; there is no CPU path")
+    out = torch.empty((tokens, v), dtype=proj.dtype, device=proj.device)
+    _lib.call("pylon_gla_recurrent", _dev(out, "out"), proj.data_ptr(), dtype_code(proj.dtype),
+              proj.stride(0) if tokens > 1 else proj.shape[1], 0, q, 2 * q, 2 * q + v, 2 * q + 2 * v, rank,
+              _dev(a2, "a2", torch.float32), _dev(a2_bias, "a2_bias", torch.float32), 1.0 / float(tau),
+              _dev(state, "state", torch.float32), _dev(norm_weight, "norm_weight", torch.float32),
+              _dev(row_start, "row_start", torch.int32), _dev(row_slots, "row_slots", torch.int32), rows, heads, dim,
+              vdim, float(eps), float(q_scale), _stream())
     return out
 
 
@@ -790,6 +882,14 @@ def gated_act(gate_up: torch.Tensor, *, alpha: float, offset: float, limit: floa
     _lib.call("pylon_gated_act", _dev(out, "out"), dtype_code(out.dtype), _dev(gate_up, "gate_up"),
               dtype_code(gate_up.dtype), tokens, two_i // 2, float(alpha), float(offset), float(limit),
               _dev(bias, "bias", torch.float32), _stream())
+    return out
+
+
+def relu2(x: torch.Tensor, *, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
+    """``max(x, 0)^2``, rounded once to ``out_dtype``."""
+    out = torch.empty(x.shape, dtype=out_dtype or x.dtype, device=x.device)
+    _lib.call("pylon_relu2", _dev(out, "out"), dtype_code(out.dtype), _dev(x, "x"), dtype_code(x.dtype), x.numel(),
+              _stream())
     return out
 
 
@@ -1225,6 +1325,13 @@ def linear_glu(x: torch.Tensor, gate_up: torch.Tensor, *, out_dtype: torch.dtype
     return silu_gate(linear(x, gate_up, out_dtype=out_dtype))
 
 
+def linear_relu2(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype) -> torch.Tensor:
+    """``max(x @ weight.T, 0)^2``.  Up to 128 rows the activation works on the product's float32 sums
+    and its result is rounded once; more bfloat16 rows: the library's product rounded first."""
+    sums = torch.float32 if x.shape[0] <= SPLIT_ROWS else out_dtype
+    return relu2(linear(x, weight, out_dtype=sums), out_dtype=out_dtype)
+
+
 def _chosen_args(rows: int, chosen: Optional[torch.Tensor], place: Optional[torch.Tensor]):
     """The optional table that also receives the chosen ids: ``chosen[place[r]] = id``."""
     if chosen is None and place is None:
@@ -1383,34 +1490,88 @@ def latent_prepare(down: torch.Tensor, cache: Optional[torch.Tensor], slot_map: 
     return q_latent, gate
 
 
+def latent_rotate(proj: torch.Tensor, q_out: torch.Tensor, cache: Optional[torch.Tensor], slot_map: Optional[torch.Tensor],
+                  *, q_off: int, n_heads: int, head_dim: int, rot_dim: int, c_off: int, kv_rank: int,
+                  c_weight: torch.Tensor, eps: float, inv_freq: Optional[torch.Tensor], rot_scale: float,
+                  interleaved: bool, positions: torch.Tensor) -> None:
+    """From a projection's rows (q's heads as ``[head_dim | rot_dim]`` each from ``q_off``; from ``c_off``
+    a latent of ``kv_rank`` numbers and behind it a key part of ``rot_dim`` shared by the heads): the
+    rotated part of every head of q into the last ``rot_dim`` elements of ``q_out`` ``[tokens, heads,
+    kv_rank + rot_dim]`` (the others are left alone), and into the tokens' slots of ``cache`` (``[...,
+    kv_rank + rot_dim]``; None: nothing is stored) the normed latent and the rotated key part.  Norm,
+    angles and rotation in float32; ``inv_freq`` None: the parts are copied unturned."""
+    if proj.dim() != 2 or proj.stride(1) != 1 or not proj.is_cuda:
+        raise KernelError("latent_rotate takes a 2-D projection on the GPU with contiguous rows")
+    tokens, width = proj.shape
+    if q_out.shape != (tokens, n_heads, kv_rank + rot_dim) or q_out.dtype != proj.dtype:
+        raise KernelError("latent_rotate: q_out has the wrong shape or dtype")
+    if q_off + n_heads * (head_dim + rot_dim) > width or c_off + kv_rank + rot_dim > width:
+        raise KernelError("latent_rotate: q or the latent lie outside the projection's rows")
+    if inv_freq is not None and inv_freq.numel() != rot_dim // 2:
+        raise KernelError("latent_rotate: inv_freq must hold rot_dim/2 frequencies")
+    if positions.numel() != tokens or c_weight.shape != (kv_rank,):
+        raise KernelError("latent_rotate: one position per token, one norm weight per element of the latent")
+    store = cache is not None
+    if store and (slot_map is None or slot_map.numel() != tokens or cache.dtype != proj.dtype
+                  or cache.shape[-1] != kv_rank + rot_dim):
+        raise KernelError("latent_rotate: the cache must be [..., kv_rank + rot_dim] of the projection's type, one slot per token")
+    _lib.call("pylon_latent_rotate", _dev(q_out, "q_out"), _dev(cache, "cache"), proj.data_ptr(), dtype_code(proj.dtype),
+              proj.stride(0) if tokens > 1 else width, int(q_off), n_heads, head_dim, rot_dim, int(c_off), kv_rank,
+              _dev(c_weight, "c_weight", torch.float32), float(eps), _dev(inv_freq, "inv_freq", torch.float32),
+              float(rot_scale), 1 if interleaved else 0, _dev(positions, "positions", torch.int32),
+              _dev(slot_map if store else None, "slot_map", torch.int32), tokens, 1 if store else 0, _stream())
+
+
 HEAD_PROJECT_ROWS = 64  # up to this many tokens the per-head products of bfloat16 run on the engine's own kernel
 
 
-def head_project(x: torch.Tensor, m: torch.Tensor, *, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``out[t, h] = gate[t, h] * x[t, h] @ m[h]`` for ``x`` ``[tokens, heads, n_in]`` (the heads of
-    a row side by side, rows maybe apart) and ``m`` ``[heads, n_in, n_out]``; ``gate`` float32
-    ``[tokens, heads]`` or None.  float32 operands and up to 64 bfloat16 tokens: the engine's
-    kernel (float sums in the order of ``n_in``, one rounding); more bfloat16 tokens: the
-    library's batched product, then the gate."""
+def head_project(x: torch.Tensor, m: torch.Tensor, *, gate: Optional[torch.Tensor] = None,
+                 gate_logits: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``out[t, h] = gate[t, h] * x[t, h] @ m[h]`` for ``x`` ``[tokens, heads, n_in]`` and ``m`` ``[heads,
+    n_in, n_out]``; ``gate`` float32 ``[tokens, heads]`` or None, or ``gate_logits`` of ``x``'s type
+    ``[tokens, heads]`` or ``[tokens, heads * n_out]`` whose sigmoids multiply a head's outputs or every
+    output.  ``x`` and ``out`` may be parts of wider heads and rows (``out`` is made if it is not given).
+    float32 operands and up to 64 bfloat16 tokens: the engine's kernel (float sums in the order of
+    ``n_in``, one rounding); more bfloat16 tokens: the library's batched product (where every size and
+    distance is a multiple of 8 elements, or everything lies side by side), then the gate."""
     if x.dim() != 3 or m.dim() != 3 or m.shape[0] != x.shape[1] or m.shape[1] != x.shape[2]:
         raise KernelError(f"head_project: cannot multiply {tuple(x.shape)} head by head by {tuple(m.shape)}")
     tokens, heads, n_in = x.shape
     n_out = m.shape[2]
-    if x.stride(2) != 1 or x.stride(1) != n_in or not m.is_contiguous() or not x.is_cuda:
-        raise KernelError("head_project: the heads of a row lie side by side, m is contiguous, both on the GPU")
+    if x.stride(2) != 1 or x.stride(1) < n_in or not m.is_contiguous() or not x.is_cuda or not m.is_cuda:
+        raise KernelError("head_project: a head's elements lie side by side, m is contiguous, both on the GPU")
     if gate is not None and (gate.shape != (tokens, heads) or gate.dtype != torch.float32):
         raise KernelError("head_project: gate must be float32 [tokens, heads]")
-    if x.dtype == torch.bfloat16 and m.dtype == torch.bfloat16 and tokens > HEAD_PROJECT_ROWS:
+    per = 1
+    if gate_logits is not None:
+        if gate is not None or gate_logits.dim() != 2 or gate_logits.dtype != x.dtype or gate_logits.stride(1) != 1 \
+                or gate_logits.shape[0] != tokens or gate_logits.shape[1] not in (heads, heads * n_out):
+            raise KernelError("head_project: gate_logits must be [tokens, heads] or [tokens, heads * n_out] of x's type")
+        per = heads * n_out // gate_logits.shape[1]
+    if out is None:
         out = torch.empty((tokens, heads, n_out), dtype=x.dtype, device=x.device)
+    elif out.shape != (tokens, heads, n_out) or out.dtype != x.dtype or not out.is_cuda or out.stride(2) != 1 \
+            or out.stride(1) < n_out:
+        raise KernelError("head_project: out must be [tokens, heads, n_out] of x's type with heads side by side")
+    together = x.stride(1) == n_in and out.is_contiguous()
+    even = all(v % 8 == 0 for v in (n_in, n_out, x.stride(0), x.stride(1), out.stride(0), out.stride(1)))
+    if x.dtype == torch.bfloat16 and m.dtype == torch.bfloat16 and tokens > HEAD_PROJECT_ROWS and (together or even):
         torch.bmm(x.transpose(0, 1), m, out=out.transpose(0, 1))
-        if gate is not None:
-            _lib.call("pylon_gate_heads", _dev(out, "out"), dtype_code(out.dtype), _dev(gate, "gate", torch.float32),
-                      tokens * heads, n_out, _stream())
+        if gate is not None or gate_logits is not None:
+            if not out.is_contiguous():
+                raise KernelError("head_project: a gated result lies side by side")
+            if gate is not None:
+                _lib.call("pylon_gate_heads", _dev(out, "out"), dtype_code(out.dtype), _dev(gate, "gate", torch.float32),
+                          tokens * heads, n_out, _stream())
+            else:
+                sigmoid_gate_(out.view(tokens, heads * n_out), gate_logits, per=per)
         return out
-    out = torch.empty((tokens, heads, n_out), dtype=x.dtype, device=x.device)
-    _lib.call("pylon_head_project", _dev(out, "out"), x.data_ptr(), dtype_code(x.dtype),
-              x.stride(0) if tokens > 1 else heads * n_in, _dev(m, "m"), dtype_code(m.dtype),
-              _dev(gate, "gate", torch.float32), tokens, heads, n_in, n_out, _stream())
+    _lib.call("pylon_head_project", out.data_ptr(), out.stride(0) if tokens > 1 else heads * out.stride(1), out.stride(1),
+              x.data_ptr(), dtype_code(x.dtype), x.stride(0) if tokens > 1 else heads * x.stride(1), x.stride(1),
+              _dev(m, "m"), dtype_code(m.dtype), _dev(gate, "gate", torch.float32),
+              None if gate_logits is None else gate_logits.data_ptr(),
+              0 if gate_logits is None else (gate_logits.stride(0) if tokens > 1 else gate_logits.shape[1]), per, tokens,
+              heads, n_in, n_out, _stream())
     return out
 
 

@@ -13,7 +13,9 @@ norm          ``forward(x) -> y`` and ``add_forward(resid, delta, row_idx=None) 
               tensor of either), or a :class:`Normed` (such an output that is normed before it
               is added); the sum is formed in float32, stored back into
               ``resid`` (unless ``row_idx`` picks rows), and its norm is returned in
-              the activation dtype.
+              the activation dtype.  Where the stream is kept in several copies, ``resid`` is
+              ``[copies, tokens, dim]``, ``delta`` a :class:`Streamed`, and a further argument
+              ``read`` (one number per copy; None: ones) says which sum of the copies is normed.
 position      ``rotary() -> (inv_freq, rotary_dim) | None`` for encodings applied by
               rotating q and k: float32 frequencies of the pairs ``(i, i + rotary_dim/2)``
               of the first ``rotary_dim`` elements of a head; None encodes nothing.
@@ -137,6 +139,17 @@ class DepthMixed(Scaled):
     coeff: Optional[torch.Tensor] = None
 
 
+@dataclass
+class Streamed:
+    """A part's output on its way into a residual stream kept in several copies: every copy becomes
+    ``x_t <- sum_s mix[s, t] x_s + write[t] * value`` (float32 coefficients on the device, ``[copies,
+    copies]`` and ``[copies]``).  ``value`` as in :class:`Normed`."""
+
+    value: torch.Tensor
+    mix: torch.Tensor
+    write: torch.Tensor
+
+
 def summed(delta: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
     """A part's output that has not been added to the residual stream yet, as one float32
     ``[tokens, dim]`` tensor.  What a mixer or a feed-forward hands on is either a tensor of
@@ -153,6 +166,9 @@ def summed(delta: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
     if isinstance(delta, DepthMixed):
         raise TypeError("a layer's result that is mixed with the earlier layers' needs a norm that knows how "
                         "(the built-in rmsnorm does)")
+    if isinstance(delta, Streamed):
+        raise TypeError("an output that several copies of the stream take their shares of needs a norm that knows "
+                        "how (the built-in rmsnorm and layernorm do)")
     if isinstance(delta, Scaled):
         value = summed(delta.value)
         if delta.bias is not None:

@@ -20,7 +20,8 @@ from typing import Optional, Tuple
 import torch
 
 from ..config.specs import LayerSpec
-from .base import DepthMixed, Part, Scaled, requirement_list
+from ..kernels import ops
+from .base import DepthMixed, Part, Scaled, Streamed, requirement_list
 from .registry import build_part, register_part
 
 
@@ -161,5 +162,39 @@ class SandwichNormBlock(Part):
         return resid, self.feed_forward_post_norm.pending(self.feed_forward.forward(h, ctx))
 
 
+class HyperConnectionBlock(PreNormBlock):
+    """A pre-normed layer on a residual stream in ``streams`` copies: each sublayer reads one sum of them
+    (``read``), and its output changes all of them at once, every copy becoming a mix of the old ones
+    (``mix``, from the first index to the second) plus its share of the output (``write``).  Neither costs
+    a launch: the output travels as :class:`~.base.Streamed` to the next norm, whose kernel renews the
+    copies, forms the sum that is read next and norms it."""
+
+    def __init__(self, spec: LayerSpec, *, dtype: torch.dtype, device) -> None:
+        if spec.input_conv is not None or spec.sublayer_scale or spec.depth_mix is not None:
+            raise ValueError("a layer of hyper-connections has no input convolution, sublayer scales or depth mix")
+        if not 1 <= spec.streams <= ops.STREAM_COPIES:
+            raise ValueError(f"hyper-connections take 1 to {ops.STREAM_COPIES} copies of the stream, got {spec.streams}")
+        super().__init__(spec, dtype=dtype, device=device)
+        for part in (self.mixer, self.feed_forward):
+            if part is not None and hasattr(part, "defer_output_bias"):
+                part.defer_output_bias = False
+        for name in ("mixer",) if self.feed_forward is None else ("mixer", "feed_forward"):
+            self.add_param(f"{name}_read", (spec.streams,), torch.float32, device, role="vector")
+            self.add_param(f"{name}_write", (spec.streams,), torch.float32, device, role="vector")
+            self.add_param(f"{name}_mix", (spec.streams, spec.streams), torch.float32, device, role="vector")
+
+    def _streamed(self, value, name: str) -> Streamed:
+        return Streamed(value, self.params[f"{name}_mix"], self.params[f"{name}_write"])
+
+    def forward(self, resid: torch.Tensor, delta, ctx, cache, stores: bool):
+        h = self.mixer_norm.add_forward(resid, delta, read=self.params["mixer_read"])
+        pending = self._streamed(self.mixer.forward(h, ctx, cache, stores), "mixer")
+        if self.feed_forward is None:
+            return resid, pending
+        h = self.feed_forward_norm.add_forward(resid, pending, read=self.params["feed_forward_read"])
+        return resid, self._streamed(self.feed_forward.forward(h, ctx), "feed_forward")
+
+
 register_part("block", "pre_norm", PreNormBlock, replace=True)
+register_part("block", "hyper_connections", HyperConnectionBlock, replace=True)
 register_part("block", "sandwich_norm", SandwichNormBlock, replace=True)

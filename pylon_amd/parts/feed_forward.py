@@ -1,10 +1,11 @@
-"""Gated feed-forward, gate and up fused into one matrix
-(/root/reference/src/pylon/model/layers.py:13-27): ``down(silu(gate(h)) * up(h))``."""
+"""Feed-forwards.  Gated, gate and up fused into one matrix
+(/root/reference/src/pylon/model/layers.py:13-27): ``down(silu(gate(h)) * up(h))``; plain:
+``down(act(up(h)))``."""
 from __future__ import annotations
 
 import torch
 
-from ..config.specs import CappedGatedFeedForwardSpec, GatedFeedForwardSpec
+from ..config.specs import CappedGatedFeedForwardSpec, GatedFeedForwardSpec, PlainFeedForwardSpec
 from ..kernels import ops, plan
 from .base import Part
 from .registry import register_part
@@ -71,5 +72,24 @@ class CappedGatedFeedForward(Part):
         return ops.linear_for_residual(hidden, self.params["down"], out_dtype=self.dtype)
 
 
+class PlainFeedForward(Part):
+    """``down(max(up(h), 0)^2)``.  Up to 128 rows the activation works on the float32 sums of the
+    product and its result is rounded once; beyond, the library's product is rounded first."""
+
+    def __init__(self, spec: PlainFeedForwardSpec, *, dtype: torch.dtype, device) -> None:
+        super().__init__()
+        if spec.activation != "relu2":
+            raise ValueError(f"activation {spec.activation!r} is not supported (only 'relu2')")
+        self.spec = spec
+        self.dtype = dtype
+        self.add_param("up", (spec.intermediate_size, spec.hidden_size), dtype, device)
+        self.add_param("down", (spec.hidden_size, spec.intermediate_size), dtype, device)
+
+    def forward(self, h: torch.Tensor, ctx) -> torch.Tensor:
+        hidden = ops.linear_relu2(h, self.params["up"], out_dtype=self.dtype)
+        return ops.linear_for_residual(hidden, self.params["down"], out_dtype=self.dtype)
+
+
+register_part("feed_forward", "plain_mlp", PlainFeedForward, replace=True)
 register_part("feed_forward", "gated_mlp", GatedFeedForward, replace=True)
 register_part("feed_forward", "capped_gated_mlp", CappedGatedFeedForward, replace=True)

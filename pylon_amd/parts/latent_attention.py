@@ -7,13 +7,20 @@ puts ``c`` into the token's cache slot; ``q = W_uq c_q``.  Per head ``k_j = W_uk
 ``v_j = W_uv c_j``, so ``q . k_j = (W_uk^T q) . c_j`` and ``sum_j p_j v_j = W_uv (sum_j p_j c_j)``:
 the queries are carried into the latent's space head by head, attention runs over the cached
 latents themselves (one key/value head that all query heads share, keys and values the same
-tensor), and the result is carried to the value space head by head, multiplied by the head's gate.
-No positions are encoded; the mask is a sliding window, chunks, or plain causal.
+tensor), and the result is carried to the value space head by head, multiplied by the gate.
+The mask is a sliding window, chunks, or plain causal.
 
-The cache is ``[pages, page_size, 1, kv_rank]`` per run (``KVRequirement(values=False)``).
-bfloat16 steps over latents of 64, 128 or 256 numbers run on the matrix-core attention kernels
-(for a step of single tokens the heads are handed to the decode kernel in groups of at most 16,
-each group as a query token of its own); everything else on the general kernel.
+Without a query latent (``q_rank`` None) the one product is ``[q; c'; r'; g]``, and a part of every
+query may carry the token's position: with ``rot_dim`` a head of q is ``[q_u | q_r]``, ``q_r`` and one
+key part ``r'`` shared by all heads are rotated, and ``q . k_j = q_u . (W_uk c_j) + q_r . r_j = [W_uk^T
+q_u | q_r] . [c_j | r_j]``: still one product over a row of the cache, whose first ``kv_rank`` elements
+are the values.  The softmax may have a learned sink per head; the gate is one number per head or per
+element.
+
+The cache is ``[pages, page_size, 1, kv_rank + rot_dim]`` per run (``KVRequirement(values=False)``).
+Without a rotated part and a sink, bfloat16 steps over latents of 64, 128 or 256 numbers run on the
+matrix-core attention kernels (for a step of single tokens the heads are handed to the decode kernel
+in groups of at most 16, each group as a query token of its own); everything else on the general kernel.
 """
 from __future__ import annotations
 
@@ -22,7 +29,7 @@ import torch
 from ..config.specs import LatentAttentionSpec
 from ..kernels import ops
 from .base import KVRequirement, Part
-from .registry import register_part
+from .registry import build_part, register_part
 
 
 def head_group(n_heads: int, most: int = 16) -> int:
@@ -33,30 +40,52 @@ def head_group(n_heads: int, most: int = 16) -> int:
 class LatentAttention(Part):
     def __init__(self, spec: LatentAttentionSpec, *, dtype: torch.dtype, device) -> None:
         super().__init__()
-        for name in ("n_heads", "head_dim", "v_head_dim", "q_rank", "kv_rank"):
+        for name in ("n_heads", "head_dim", "v_head_dim", "kv_rank"):
             if getattr(spec, name) < 1:
                 raise ValueError(f"latent attention: {name} must be positive")
+        if spec.q_rank is not None and spec.q_rank < 1:
+            raise ValueError("latent attention: q_rank must be positive (or None)")
+        if spec.rot_dim < 0 or spec.rot_dim % 2 or spec.rot_dim > 512:
+            raise ValueError("latent attention: rot_dim must be even, at most 512")
+        if spec.q_rank is not None and (spec.rot_dim or spec.gate_over != "head"):
+            raise ValueError("a rotated part and gates per element go with queries straight from the input")
         if spec.kv_rank > 512:
             raise ValueError(f"a latent of {spec.kv_rank} numbers is not supported: the attention kernels take up to 512")
         if spec.window is not None and spec.window < 1:
             raise ValueError("window must be positive (or None)")
         if spec.chunk is not None and (spec.chunk < 1 or spec.window is not None):
             raise ValueError("chunk must be positive, and a layer has a window or chunks, not both")
+        if spec.gate_over not in ("head", "element"):
+            raise ValueError(f"gate_over must be 'head' or 'element', got {spec.gate_over!r}")
         self.spec = spec
         self.dtype = dtype
-        self.n_gate = spec.n_heads if spec.gate else 0
-        self.add_param("down", (spec.q_rank + spec.kv_rank + self.n_gate, spec.hidden_size), dtype, device)
-        self.add_param("q_norm", (spec.q_rank,), torch.float32, device, role="vector")
+        self.n_gate = spec.gate_size
+        # the rows of the one product over the input: q (or its latent), the latent, the shared rotated
+        # key part, the gate
+        self.q_rows = spec.n_heads * (spec.head_dim + spec.rot_dim) if spec.q_rank is None else spec.q_rank
+        self.gate_off = self.q_rows + spec.kv_rank + spec.rot_dim
+        self.width = spec.kv_rank + spec.rot_dim  # a row of the cache
+        self.add_param("down", (self.gate_off + self.n_gate, spec.hidden_size), dtype, device)
         self.add_param("c_norm", (spec.kv_rank,), torch.float32, device, role="vector")
-        self.add_param("uq", (spec.n_heads * spec.head_dim, spec.q_rank), dtype, device)
+        if spec.q_rank is not None:
+            self.add_param("q_norm", (spec.q_rank,), torch.float32, device, role="vector")
+            self.add_param("uq", (spec.n_heads * spec.head_dim, spec.q_rank), dtype, device)
         self.add_param("uk", (spec.n_heads * spec.head_dim, spec.kv_rank), dtype, device)
         self.add_param("uv", (spec.n_heads * spec.v_head_dim, spec.kv_rank), dtype, device)
         self.add_param("out", (spec.hidden_size, spec.n_heads * spec.v_head_dim), dtype, device)
+        if spec.sink:
+            self.add_param("sink", (spec.n_heads,), torch.float32, device, role="vector")
+        self.position = None
+        if spec.rot_dim and spec.position is not None:
+            self.position = self.add_child("position", build_part("position", spec.position, dtype=dtype, device=device))
+            rotary = self.position.rotary()
+            if rotary is not None and rotary[1] != spec.rot_dim:
+                raise ValueError(f"latent attention rotates its whole part of {spec.rot_dim} elements, not {rotary[1]}")
         self._uv_by_latent = None  # (version of uv, uv as [heads, kv_rank, v_head_dim])
 
     def cache_requirement(self) -> KVRequirement:
         spec = self.spec
-        return KVRequirement(1, spec.kv_rank, spec.window, chunk=spec.chunk, values=False)
+        return KVRequirement(1, self.width, spec.window, chunk=spec.chunk, values=False)
 
     def value_maps(self) -> torch.Tensor:
         """``uv`` with the latent's axis first inside every head, ``[heads, kv_rank, v_head_dim]``:
@@ -89,7 +118,9 @@ class LatentAttention(Part):
         return head_group(self.spec.n_heads, 8 if self.spec.kv_rank >= 256 else 16)
 
     def _matrix_cores(self) -> bool:
-        return self.dtype == torch.bfloat16 and self.spec.kv_rank in ops.DECODE_HEAD_DIMS
+        spec = self.spec
+        return (self.dtype == torch.bfloat16 and spec.kv_rank in ops.DECODE_HEAD_DIMS and not spec.rot_dim
+                and not spec.sink)
 
     def decode_signature(self, rows: int, bound: int) -> tuple:
         if not self._matrix_cores():
@@ -101,16 +132,49 @@ class LatentAttention(Part):
         spec = self.spec
         tokens = h.shape[0]
         heads, rank = spec.n_heads, spec.kv_rank
-        down = ops.linear(h, self.params["down"], out_dtype=torch.float32)
-        q_latent, gate = ops.latent_prepare(
-            down, cache.k if stores else None, cache.slot_map if stores else None, q_rank=spec.q_rank,
-            kv_rank=rank, n_gate=self.n_gate, q_weight=self.params["q_norm"], c_weight=self.params["c_norm"],
-            eps=spec.norm_eps, out_dtype=self.dtype)
-        q = ops.linear(q_latent, self.params["uq"], out_dtype=self.dtype)
-        # the queries in the latent's space: q'_h = W_uk[h]^T q_h
-        q = ops.head_project(q.view(tokens, heads, spec.head_dim), self.params["uk"].view(heads, spec.head_dim, rank))
+        gating = {}
+        if spec.q_rank is None:
+            q, gating["gate_logits"] = self._queries(h, ctx, cache, stores)
+        else:
+            down = ops.linear(h, self.params["down"], out_dtype=torch.float32)
+            q_latent, gating["gate"] = ops.latent_prepare(
+                down, cache.k if stores else None, cache.slot_map if stores else None, q_rank=spec.q_rank,
+                kv_rank=rank, n_gate=self.n_gate, q_weight=self.params["q_norm"], c_weight=self.params["c_norm"],
+                eps=spec.norm_eps, out_dtype=self.dtype)
+            q = ops.linear(q_latent, self.params["uq"], out_dtype=self.dtype)
+            # the queries in the latent's space: q'_h = W_uk[h]^T q_h
+            q = ops.head_project(q.view(tokens, heads, spec.head_dim), self.params["uk"].view(heads, spec.head_dim, rank))
+        mixed = self._attend(q, ctx, cache)
+        # to the value space head by head, times the gate
+        context = ops.head_project(mixed, self.value_maps(), **gating)
+        return ops.linear_for_residual(context.view(tokens, heads * spec.v_head_dim), self.params["out"],
+                                       out_dtype=self.dtype)
+
+    def _queries(self, h: torch.Tensor, ctx, cache, stores: bool):
+        """``(queries in the cache rows' space [tokens, heads, kv_rank + rot_dim], the gate's logits or
+        None)`` of queries that come straight from the input; the tokens' rows go into the cache."""
+        spec = self.spec
+        tokens, heads, rank = h.shape[0], spec.n_heads, spec.kv_rank
+        proj = ops.linear(h, self.params["down"], out_dtype=self.dtype)
+        q = torch.empty((tokens, heads, self.width), dtype=self.dtype, device=h.device)
+        rotary = self.position.rotary() if self.position is not None else None
+        ops.latent_rotate(
+            proj, q, cache.k if stores else None, cache.slot_map if stores else None, q_off=0, n_heads=heads,
+            head_dim=spec.head_dim, rot_dim=spec.rot_dim, c_off=self.q_rows, kv_rank=rank, c_weight=self.params["c_norm"],
+            eps=spec.norm_eps, inv_freq=rotary[0] if rotary else None,
+            rot_scale=self.position.rot_scale if rotary else 1.0,
+            interleaved=self.position.interleaved if rotary else True, positions=ctx.positions)
+        unrotated = proj[:, : self.q_rows].view(tokens, heads, spec.head_dim + spec.rot_dim)[..., : spec.head_dim]
+        ops.head_project(unrotated, self.params["uk"].view(heads, spec.head_dim, rank), out=q[..., :rank])
+        return q, proj[:, self.gate_off:] if self.n_gate else None
+
+    def _attend(self, q: torch.Tensor, ctx, cache) -> torch.Tensor:
+        """``[tokens, heads, kv_rank]``: every head's weighted sum of its request's latents."""
+        spec = self.spec
+        tokens, heads, width = q.shape
+        rank = spec.kv_rank
         mask = dict(window=spec.window, chunk=spec.chunk)
-        latents = cache.k  # [pages, page_size, 1, kv_rank]: keys and values at once
+        latents = cache.k  # [pages, page_size, 1, kv_rank + rot_dim]: keys, and values at their front
         group = self._group()
         repeat = heads // group
         if self._matrix_cores() and q.dtype == latents.dtype and ctx.decode_only \
@@ -122,23 +186,19 @@ class LatentAttention(Part):
                     ctx.memo[key] = (ctx.positions.repeat_interleave(repeat), ctx.tok_row.repeat_interleave(repeat))
                 positions, rows = ctx.memo[key]
             cuts, splits = self._decode_launch(tokens * repeat, self._span(ctx.max_len))
-            mixed = ops.attention_decode(
+            return ops.attention_decode(
                 q.view(tokens * repeat, group, rank), latents, latents, cache.block_table, rows, positions,
                 page_size=cache.page_size, scale=spec.scale, n_splits=splits, n_cuts=cuts, **mask,
             ).view(tokens, heads, rank)
-        elif self._matrix_cores() and q.dtype == latents.dtype and ops.prefill_attention_ok(q, latents, cache.block_table):
+        if self._matrix_cores() and q.dtype == latents.dtype and ops.prefill_attention_ok(q, latents, cache.block_table):
             rows = ops.prefill_rows(tokens, heads, heads)
             mixed = torch.empty_like(q)
             tiles = ctx.token_tiles(rows // heads, fold=ops.prefill_fold(1))
-            ops.attention_prefill(q, latents, latents, cache.block_table, tiles, page_size=cache.page_size,
-                                  scale=spec.scale, rows=rows, out=mixed, **mask)
-        else:
-            mixed = ops.paged_attention(q, latents, latents, cache.block_table, ctx.tok_row, ctx.positions,
-                                        page_size=cache.page_size, scale=spec.scale, **mask)
-        # to the value space head by head, times the head's gate
-        context = ops.head_project(mixed, self.value_maps(), gate=gate)
-        return ops.linear_for_residual(context.view(tokens, heads * spec.v_head_dim), self.params["out"],
-                                       out_dtype=self.dtype)
+            return ops.attention_prefill(q, latents, latents, cache.block_table, tiles, page_size=cache.page_size,
+                                         scale=spec.scale, rows=rows, out=mixed, **mask)
+        return ops.paged_attention(q, latents, latents, cache.block_table, ctx.tok_row, ctx.positions,
+                                   page_size=cache.page_size, scale=spec.scale, values_in_keys=rank,
+                                   sink_logit=self.params.get("sink"), **mask)
 
 
 register_part("mixer", "latent_attention", LatentAttention, replace=True)

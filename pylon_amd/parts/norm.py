@@ -1,7 +1,8 @@
-"""RMSNorm over the hidden axis (/root/reference/src/pylon/model/layers.py:30-40):
+"""Norms over the hidden axis.  RMSNorm (/root/reference/src/pylon/model/layers.py:30-40):
 ``y = x / sqrt(mean(x^2) + eps) * w`` in float32, rounded once to the activation dtype.
 The weight is kept in float32 whatever the model's dtype, as the reference keeps it.  With
-``weight_offset`` the stored weight is a distance from that number: ``y = ... * (offset + w)``."""
+``weight_offset`` the stored weight is a distance from that number: ``y = ... * (offset + w)``.
+LayerNorm subtracts the mean first and divides by the root mean square of the deviations."""
 from __future__ import annotations
 
 from typing import Optional
@@ -10,7 +11,7 @@ import torch
 
 from ..config.specs import NormSpec
 from ..kernels import ops
-from .base import DepthMixed, Normed, Part, Scaled
+from .base import DepthMixed, Normed, Part, Scaled, Streamed, summed
 from .registry import register_part
 
 
@@ -36,8 +37,10 @@ class RMSNorm(Part):
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         return ops.rmsnorm(x, self.weight(), self.spec.eps, out_dtype=self.dtype)
 
-    def add_forward(self, resid: torch.Tensor, delta, *,
-                    row_idx: Optional[torch.Tensor] = None) -> torch.Tensor:
+    def add_forward(self, resid: torch.Tensor, delta, *, row_idx: Optional[torch.Tensor] = None,
+                    read: Optional[torch.Tensor] = None) -> torch.Tensor:
+        if resid.dim() == 3 or isinstance(delta, Streamed) or read is not None:
+            return _copies_forward(self, resid, delta, row_idx, read, centre=False)
         if isinstance(delta, Normed):
             return ops.add_normed_rmsnorm(resid, delta.value, self.weight(), self.spec.eps, self.dtype,
                                           post_gain=delta.gain, post_eps=delta.eps, row_idx=row_idx)
@@ -55,6 +58,44 @@ class RMSNorm(Part):
                                           row_idx=row_idx, delta_scale=delta.scale, delta_bias=delta.bias)
         return ops.add_rmsnorm(resid, delta, self.weight(), self.spec.eps, self.dtype,
                                row_idx=row_idx)
+
+
+def _copies_forward(norm, resid: torch.Tensor, delta, row_idx, read, *, centre: bool) -> torch.Tensor:
+    """The norm over a residual stream in several copies (or one): what the last sublayer left for them,
+    and the sum of them that is normed, in one kernel."""
+    if isinstance(delta, Streamed):
+        return ops.stream_norm(resid, delta.value, norm.weight(), norm.spec.eps, norm.dtype, centre=centre, mix=delta.mix,
+                               write=delta.write, read=read, row_idx=row_idx)
+    if resid.dim() == 3 and delta is not None:
+        raise TypeError("an output for a stream in several copies comes with their shares of it (Streamed)")
+    if delta is not None and not isinstance(delta, torch.Tensor):
+        delta = summed(delta)
+    return ops.stream_norm(resid, delta, norm.weight(), norm.spec.eps, norm.dtype, centre=centre, read=read,
+                           row_idx=row_idx)
+
+
+class LayerNorm(Part):
+    """``(x - mean(x)) / sqrt(mean((x - mean(x))^2) + eps) * w`` in float32, rounded once to the
+    activation dtype; a weight in float32, no bias."""
+
+    def __init__(self, spec: NormSpec, *, dtype: torch.dtype, device) -> None:
+        super().__init__()
+        self.spec = spec
+        self.dtype = dtype
+        if spec.weight_offset:
+            raise ValueError("a layer norm's weights are stored as they are")
+        self.add_param("weight", (spec.dim,), torch.float32, device, role="vector")
+
+    def weight(self) -> torch.Tensor:
+        return self.params["weight"]
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return ops.stream_norm(x.float() if x.dtype != torch.float32 else x, None, self.params["weight"], self.spec.eps,
+                               self.dtype, centre=True)
+
+    def add_forward(self, resid: torch.Tensor, delta, *, row_idx: Optional[torch.Tensor] = None,
+                    read: Optional[torch.Tensor] = None) -> torch.Tensor:
+        return _copies_forward(self, resid, delta, row_idx, read, centre=True)
 
 
 class ScalarRMSNorm(Part):
@@ -84,4 +125,5 @@ class ScalarRMSNorm(Part):
 
 
 register_part("norm", "rmsnorm", RMSNorm, replace=True)
+register_part("norm", "layernorm", LayerNorm, replace=True)
 register_part("norm", "scalar_rmsnorm", ScalarRMSNorm, replace=True)

@@ -905,7 +905,7 @@ def test_kernels_refuse_what_they_cannot_do(ops):
     from pylon_amd.kernels import KernelError
 
     q = torch.zeros((1, 2, 520), device=DEV)
-    kc = torch.zeros((2, 16, 1, 520), device=DEV)
+    kc = torch.zeros((2, 16, 1, 1032), device=DEV)
     z = torch.zeros(1, dtype=torch.int32, device=DEV)
     with pytest.raises(KernelError, match="between 1 and 512"):
         ops.paged_attention(q, kc, kc, torch.zeros((1, 1), dtype=torch.int32, device=DEV), z, z,
