@@ -2,7 +2,7 @@
 and uniform-random token ids, on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--layers L]
-                    [--shape 4b|8b|32b] [--prompt-len N] [--design vupuzen|pavitar|gimudra|tukarax [--beside qwen3|vupuzen|pavitar|gimudra] [--design-shapes 8b,...]]
+                    [--shape 4b|8b|32b] [--prompt-len N] [--design vupuzen|pavitar|gimudra|tukarax|ranudra [--beside qwen3|vupuzen|pavitar|gimudra] [--design-shapes 8b,...]]
 
 Everything goes the product's own way.  Start-up is ``Runner.from_random``: the fit check,
 the measured activation headroom, the page pool sized from the card's memory and the decode
@@ -381,6 +381,30 @@ def tukarax_json(shape: dict, layers: int) -> dict:
             "layers": [parallel if i % 2 == 0 else attention for i in range(layers)]}
 
 
+def ranudra_json(shape: dict, layers: int) -> dict:
+    """A Ranudra configuration of the shape's layer sizes: of every three layers one gated linear
+    attention (as many heads of the shape's head size as fill half the width) and one of each kind of
+    latent attention (the shape's heads, 64 rotated elements besides those of a head, a latent of 256
+    numbers, windows of 1,024 positions); a plain feed-forward as large as the shape's gated one (its
+    three matrices as two); a residual stream in two copies; the shape's vocabulary.  Of ``layers`` runs
+    the middle stretch runs twice over the same weights (a quarter fewer layers own weights)."""
+    width, hd, heads = shape["hidden_size"], shape["head_dim"], shape["num_attention_heads"]
+    mlp = {"kind": "dense", "ff": shape["intermediate_size"] * 3 // 2}
+    linear = {"type": "gla", "mixer": {"heads": max(1, width // (2 * hd)), "dim": hd, "vdim": hd, "tau": 16.0}, "mlp": mlp}
+    sizes = {"heads": heads, "dim": hd, "rot_dim": 64, "vdim": hd, "kv_rank": 256, "scale": (hd + 64) ** -0.5,
+             "mask": {"size": 1024}}
+    first = {"type": "latent_attention", "mlp": mlp, "mixer": {**sizes, "rot": {
+        "base": 1000000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    second = {"type": "latent_attention_2", "mlp": mlp, "mixer": {**sizes, "rot": {"base": 250000.0, "dims": 64}}}
+    again = layers // 4  # this many layers run twice
+    own = layers - again
+    start = (own - again) // 2
+    return {"architecture": "Ranudra", "vocab": shape["vocab_size"], "width": width, "streams": 2,
+            "embedding": {"scale": 16.0}, "norm": {"eps": 1e-6},
+            "loop": {"start": start, "stop": start + again, "times": 2} if again else None,
+            "layers": [(linear, first, second)[i % 3] for i in range(own)]}
+
+
 def design_steps(runner, vocab: int, batch: int, prompt_len: int, steps: int, warmup: int, seed: int) -> dict:
     """Milliseconds of one prompt step of ``prompt_len`` tokens (median of five), and of a
     decode step of ``batch`` requests behind such prompts (mean of ``steps``), through the step
@@ -422,7 +446,7 @@ def design_steps(runner, vocab: int, batch: int, prompt_len: int, steps: int, wa
 
 
 def design_main(args) -> int:
-    """``--design vupuzen|pavitar|gimudra|tukarax``: prefill and decode of models of that design of random
+    """``--design vupuzen|pavitar|gimudra|tukarax|ranudra``: prefill and decode of models of that design of random
     weights at the layer sizes of ``--shape`` (and of the other shapes named by ``--design-shapes``),
     beside the model of the design ``--beside`` (Qwen3 unless told otherwise) of the same sizes and
     number of layer runs, both through the same step function over pages of 256 tokens with decode
@@ -444,7 +468,7 @@ def design_main(args) -> int:
         layers = args.layers or 8
         pages = (args.batch + 1) * (-(-(prompt_len + steps + warmup + 8) // PAGE_SIZE) + 1)
         makers = {"vupuzen": vupuzen_json, "pavitar": pavitar_json, "gimudra": gimudra_json, "tukarax": tukarax_json,
-                  "qwen3": config_json}
+                  "ranudra": ranudra_json, "qwen3": config_json}
         for design, raw in ((args.design, makers[args.design](shape, layers)), (beside, makers[beside](shape, layers))):
             config = PylonConfig(dtype=args.dtype, max_batch_size=args.batch + 1, max_queue_size=args.batch + 1,
                                  page_size=PAGE_SIZE, prefill_chunk_size=prompt_len, num_pages=pages,
@@ -495,9 +519,9 @@ def main() -> int:
     parser.add_argument("--no-peaks", action="store_true", help="skip the probes of this device's own peaks")
     parser.add_argument("--mixed", action="store_true",
                         help="also time a step of --batch decoded tokens beside a 2,048-token prompt portion")
-    parser.add_argument("--design", choices=("qwen3", "vupuzen", "pavitar", "gimudra", "tukarax"), default="qwen3",
-                        help="vupuzen, pavitar, gimudra, tukarax: that design beside Qwen3 at equal sizes instead of the default workload")
-    parser.add_argument("--beside", choices=("qwen3", "vupuzen", "pavitar", "gimudra"), default="qwen3",
+    parser.add_argument("--design", choices=("qwen3", "vupuzen", "pavitar", "gimudra", "tukarax", "ranudra"), default="qwen3",
+                        help="vupuzen, pavitar, gimudra, tukarax, ranudra: that design beside Qwen3 at equal sizes instead of the default workload")
+    parser.add_argument("--beside", choices=("qwen3", "vupuzen", "pavitar", "gimudra", "tukarax"), default="qwen3",
                         help="with another --design: the design it is measured beside (default qwen3)")
     parser.add_argument("--design-shapes", default="", help="with another --design: further shapes, with commas")
     parser.add_argument("--prefill-only", action="store_true",

@@ -42,6 +42,7 @@ HIPCC_FLAGS = [
 # extra moves, and the kernel needs fewer registers in total this way).
 EXTRA_FLAGS = {
     "attention_prefill.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"],
+    "attention_latent.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"],
 }
 
 

@@ -61,6 +61,9 @@ _SIGNATURES = {
     "pylon_sample": [P, P, I, I, L, P, P, P, P, P, P],
     "pylon_qkv_prepare_wide": [P, P, P, P, I, L, P, P, F, P, I, I, P, P, I, I, I, I, I, I, I, F, I, I, P],
     "pylon_latent_prepare": [P, P, P, P, L, I, P, P, F, P, I, I, I, I, I, P],
+    "pylon_latent_attention_ok": [I, I, I],
+    "pylon_latent_prefill": [P, P, P, P, I, P, I, I, I, I, I, I, F, P, I, P],
+    "pylon_latent_decode": [P, P, P, P, I, P, I, I, I, I, I, I, F, P, I, P, L, P],
     "pylon_latent_rotate": [P, P, P, I, L, I, I, I, I, I, I, P, F, P, F, I, P, P, I, I, P],
     "pylon_head_project": [P, L, I, P, I, L, I, P, I, P, P, L, I, I, I, I, I, P],
     "pylon_gate_heads": [P, I, P, L, I, P],

@@ -683,6 +683,15 @@ def gla_recurrent(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_
     return out
 
 
+def gla(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_bias: torch.Tensor, norm_weight: torch.Tensor,
+        row_start: torch.Tensor, row_slots: torch.Tensor, *, rows: int, heads: int, dim: int, vdim: int, rank: int,
+        tau: float, eps: float, q_scale: float, max_count: int) -> torch.Tensor:
+    """Gated linear attention over the rows of a step (:func:`gla_recurrent` says what it computes);
+    ``max_count`` is the most tokens a row brings."""
+    return gla_recurrent(proj, state, a2, a2_bias, norm_weight, row_start, row_slots, rows=rows, heads=heads, dim=dim,
+                         vdim=vdim, rank=rank, tau=tau, eps=eps, q_scale=q_scale)
+
+
 def kv_store(proj: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, slot_map: torch.Tensor, *,
              k_off: int, v_off: int, v_transposed: bool = False) -> None:
     """Copy every token's keys (``proj[t, k_off:]``) and values (``proj[t, v_off:]``) into its
@@ -1520,6 +1529,101 @@ def latent_rotate(proj: torch.Tensor, q_out: torch.Tensor, cache: Optional[torch
               _dev(c_weight, "c_weight", torch.float32), float(eps), _dev(inv_freq, "inv_freq", torch.float32),
               float(rot_scale), 1 if interleaved else 0, _dev(positions, "positions", torch.int32),
               _dev(slot_map if store else None, "slot_map", torch.int32), tokens, 1 if store else 0, _stream())
+
+
+_LATENT_SHAPES = ((64, 64), (96, 64), (128, 128), (192, 128), (256, 128), (320, 256), (384, 256), (576, 512))
+
+
+def latent_attention_ok(dtype: torch.dtype, *, width: int, rank: int, page_size: int) -> bool:
+    """Whether the matrix-core kernels over cached rows of ``width`` elements whose first ``rank`` are the
+    values take this geometry (the kernels' own rule)."""
+    return (dtype == torch.bfloat16 and width % 8 == 0 and 1 <= rank <= width and page_size % 64 == 0
+            and any(width <= w and rank <= r for w, r in _LATENT_SHAPES))
+
+
+def latent_rows(tokens: int, n_heads: int, rank: int) -> Optional[int]:
+    """Query rows of a workgroup of :func:`latent_prefill`: 128 halve the traffic from LDS per matrix
+    instruction, a step with few query rows fills more of the chip with workgroups of 64; values of more
+    than 256 elements leave registers for 64 only.  None: more heads than a workgroup takes."""
+    if rank > 256:
+        return 64 if n_heads <= 64 else None
+    if n_heads > 64:
+        return 128 if n_heads <= 128 else None
+    return 128 if tokens * n_heads >= 128 * 256 else 64
+
+
+def _latent_checks(name: str, q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor, rank: int,
+                   page_size: int, sink: Optional[torch.Tensor]) -> None:
+    if q.dim() != 3 or cache.dim() != 4 or cache.shape[2] != 1 or cache.shape[3] != q.shape[2] \
+            or cache.shape[1] != page_size or cache.dtype != q.dtype:
+        raise KernelError(f"{name}: q is [tokens, heads, width] and the cache [pages, page_size, 1, width] of its type")
+    if not latent_attention_ok(q.dtype, width=q.shape[2], rank=rank, page_size=page_size):
+        raise KernelError(f"{name} does not take this geometry")
+    if cache.shape[0] * page_size >= 2 ** 31 or block_table.dim() != 2:
+        raise KernelError(f"{name}: the cache is too large for int32 slots, or the table is not 2-D")
+    if sink is not None and sink.shape != (q.shape[1],):
+        raise KernelError(f"{name}: sink is float32 [heads]")
+
+
+def latent_prefill(q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor, tiles: torch.Tensor, *, rank: int,
+                   page_size: int, scale: float, rows: int, window: Optional[int] = None, chunk: Optional[int] = None,
+                   sink: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Causal attention of bfloat16 prompt portions over cached rows that all heads share (``cache``
+    ``[pages, page_size, 1, width]``; a row is a key, its first ``rank`` elements the value) on the matrix
+    cores: ``[tokens, heads, rank]``.  ``tiles`` int32 ``[n, 4]``: first token, count, block-table row and
+    first position of runs of at most ``rows // heads`` consecutive tokens of one request; tokens that no
+    tile covers are left as they are in ``out``.  ``sink`` float32 ``[heads]``: ``exp(sink)`` joins the
+    denominator.  Masks as in :func:`mask_code`."""
+    _latent_checks("latent_prefill", q, cache, block_table, rank, page_size, sink)
+    tokens, n_heads, width = q.shape
+    if tiles.dim() != 2 or tiles.shape[1] != 4:
+        raise KernelError("latent_prefill: tiles must be [n, 4]")
+    if out is None:
+        out = torch.empty((tokens, n_heads, rank), dtype=q.dtype, device=q.device)
+    elif out.shape != (tokens, n_heads, rank) or out.dtype != q.dtype:
+        raise KernelError("latent_prefill: out must be [tokens, heads, rank] of q's type")
+    _lib.call("pylon_latent_prefill", _dev(out, "out"), _dev(q, "q"), _dev(cache, "cache"),
+              _dev(block_table, "block_table", torch.int32), block_table.shape[1], _dev(tiles, "tiles", torch.int32),
+              tiles.shape[0], n_heads, width, rank, page_size, mask_code(window, chunk), float(scale),
+              _dev(sink, "sink", torch.float32), int(rows), _stream())
+    return out
+
+
+def latent_cuts(tokens: int, n_heads: int, span: int, units: Optional[int] = None) -> int:
+    """Workgroups that share the keys of one token and group of heads in a step of single tokens: more
+    while the launch leaves compute units idle and every cut keeps 128 keys, a block for each wave."""
+    units = units or _lib.compute_units()
+    groups = tokens * (-(-n_heads // (32 if n_heads > 16 else 16)))
+    cuts = 1
+    while cuts < 64 and groups * cuts * 2 <= units and cuts * 2 * 128 <= span:
+        cuts *= 2
+    return cuts
+
+
+def latent_decode(q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor, positions: torch.Tensor, *, rank: int,
+                  page_size: int, scale: float, cuts: int = 1, window: Optional[int] = None,
+                  chunk: Optional[int] = None, sink: Optional[torch.Tensor] = None,
+                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """:func:`latent_prefill` for a step of single tokens: token ``t`` is on row ``t`` of the block table
+    at ``positions[t]``; ``cuts`` workgroups share a token's keys and a second kernel merges their
+    float32 partial results."""
+    _latent_checks("latent_decode", q, cache, block_table, rank, page_size, sink)
+    tokens, n_heads, width = q.shape
+    if positions.numel() != tokens or block_table.shape[0] < tokens:
+        raise KernelError("latent_decode: one position and one row of the table per token")
+    if out is None:
+        out = torch.empty((tokens, n_heads, rank), dtype=q.dtype, device=q.device)
+    elif out.shape != (tokens, n_heads, rank) or out.dtype != q.dtype:
+        raise KernelError("latent_decode: out must be [tokens, heads, rank] of q's type")
+    partial = None
+    if cuts > 1:
+        partial = torch.empty((tokens * n_heads * cuts * (2 + rank),), dtype=torch.float32, device=q.device)
+    _lib.call("pylon_latent_decode", _dev(out, "out"), _dev(q, "q"), _dev(cache, "cache"),
+              _dev(block_table, "block_table", torch.int32), block_table.shape[1],
+              _dev(positions, "positions", torch.int32), tokens, n_heads, width, rank, page_size,
+              mask_code(window, chunk), float(scale), _dev(sink, "sink", torch.float32), int(cuts),
+              _dev(partial, "partial"), 0 if partial is None else partial.numel(), _stream())
+    return out
 
 
 HEAD_PROJECT_ROWS = 64  # up to this many tokens the per-head products of bfloat16 run on the engine's own kernel

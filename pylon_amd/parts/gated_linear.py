@@ -46,10 +46,11 @@ class GatedLinearAttention(Part):
         if not stores:
             raise ValueError("a gated linear attention layer cannot borrow another run's state")
         proj = ops.linear(h, self.params["proj"], out_dtype=self.dtype)
-        mixed = ops.gla_recurrent(
+        mixed = ops.gla(
             proj, cache.state, self.params["a2"], self.params["a2_bias"], self.params["norm"], ctx.row_start,
             ctx.row_slots, rows=ctx.rows, heads=spec.n_heads, dim=spec.head_dim, vdim=spec.v_head_dim,
-            rank=spec.decay_rank, tau=spec.tau, eps=spec.norm_eps, q_scale=spec.head_dim ** -0.5)
+            rank=spec.decay_rank, tau=spec.tau, eps=spec.norm_eps, q_scale=spec.head_dim ** -0.5,
+            max_count=ctx.max_count)
         return ops.linear_for_residual(mixed, self.params["out"], out_dtype=self.dtype)
 
 

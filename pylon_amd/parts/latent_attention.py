@@ -20,7 +20,9 @@ element.
 The cache is ``[pages, page_size, 1, kv_rank + rot_dim]`` per run (``KVRequirement(values=False)``).
 Without a rotated part and a sink, bfloat16 steps over latents of 64, 128 or 256 numbers run on the
 matrix-core attention kernels (for a step of single tokens the heads are handed to the decode kernel
-in groups of at most 16, each group as a query token of its own); everything else on the general kernel.
+in groups of at most 16, each group as a query token of its own).  With them, bfloat16 steps over
+pages of a multiple of 64 tokens run on kernels of their own (``attention_latent.hip``) that bring a block
+of rows into LDS once and read it as keys and as values.  Everything else runs on the general kernel.
 """
 from __future__ import annotations
 
@@ -124,9 +126,16 @@ class LatentAttention(Part):
 
     def decode_signature(self, rows: int, bound: int) -> tuple:
         if not self._matrix_cores():
-            return ("latent_attention",)
+            # over whole cache rows (whatever the page's size, which this does not know) the keys' cuts
+            return ("latent_attention", ops.latent_cuts(rows, self.spec.n_heads, self._span(bound)))
         group = self._group()
         return ("latent_attention",) + tuple(self._decode_launch(rows * (self.spec.n_heads // group), self._span(bound)))
+
+    def _row_kernels(self, page_size: int) -> bool:
+        """Whether the matrix-core kernels over whole cache rows (a key with its value at the front) run."""
+        spec = self.spec
+        return bool(spec.rot_dim or spec.sink) and ops.latent_attention_ok(
+            self.dtype, width=self.width, rank=spec.kv_rank, page_size=page_size)
 
     def forward(self, h: torch.Tensor, ctx, cache, stores: bool) -> torch.Tensor:
         spec = self.spec
@@ -196,6 +205,21 @@ class LatentAttention(Part):
             tiles = ctx.token_tiles(rows // heads, fold=ops.prefill_fold(1))
             return ops.attention_prefill(q, latents, latents, cache.block_table, tiles, page_size=cache.page_size,
                                          scale=spec.scale, rows=rows, out=mixed, **mask)
+        if self._row_kernels(cache.page_size) and q.dtype == latents.dtype:
+            options = dict(rank=rank, page_size=cache.page_size, scale=spec.scale, sink=self.params.get("sink"), **mask)
+            rows = ops.latent_rows(tokens, heads, rank)
+            # decoding requests at the head of a step go to the kernel of single tokens
+            singles = tokens if ctx.decode_only else (ctx.leading_singles if rows else 0)
+            if singles == tokens or rows:
+                mixed = torch.empty((tokens, heads, rank), dtype=self.dtype, device=q.device)
+                if singles:
+                    length = ctx.max_len if ctx.decode_only else int(ctx.starts[:singles].max()) + 1
+                    ops.latent_decode(q[:singles], latents, cache.block_table, ctx.positions[:singles],
+                                      cuts=ops.latent_cuts(singles, heads, self._span(length)), out=mixed[:singles], **options)
+                if singles < tokens:
+                    tiles = ctx.token_tiles(rows // heads, skip_rows=singles, fold=ops.prefill_fold(1))
+                    ops.latent_prefill(q, latents, cache.block_table, tiles, rows=rows, out=mixed, **options)
+                return mixed
         return ops.paged_attention(q, latents, latents, cache.block_table, ctx.tok_row, ctx.positions,
                                    page_size=cache.page_size, scale=spec.scale, values_in_keys=rank,
                                    sink_logit=self.params.get("sink"), **mask)
