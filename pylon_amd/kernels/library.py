@@ -38,6 +38,7 @@ _SIGNATURES = {
     "pylon_stream_norm": [P, I, P, L, I, P, I, I, L, P, P, P, P, P, I, I, F, I, P],
     "pylon_relu2": [P, I, P, I, L, P],
     "pylon_gla_recurrent": [P, P, I, L, I, I, I, I, I, I, P, P, F, P, P, P, P, I, I, I, I, F, F, P],
+    "pylon_gla_chunked": [P, P, L, I, I, I, I, I, I, P, P, F, P, P, P, P, P, I, I, I, I, F, F, I, P, L, P, L, P],
     "pylon_short_conv": [P, I, P, I, P, I, P, P, P, I, I, I, I, L, I, P],
     "pylon_token_shift": [P, I, P, I, P, P, P, P, I, I, I, P],
     "pylon_retention_recurrent": [P, P, I, L, I, I, I, I, P, P, P, I, P, P, P, I, I, I, I, F, F, P],

@@ -650,16 +650,7 @@ def gla_ok(dim: int, vdim: int) -> bool:
     return -(-dim // min(dim, 1024 // vdim)) <= 64
 
 
-def gla_recurrent(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_bias: torch.Tensor,
-                  norm_weight: torch.Tensor, row_start: torch.Tensor, row_slots: torch.Tensor, *, rows: int, heads: int,
-                  dim: int, vdim: int, rank: int, tau: float, eps: float, q_scale: float) -> torch.Tensor:
-    """Gated linear attention, token by token: ``proj`` ``[tokens, 2 heads dim + 2 heads vdim + rank]``
-    holds q, k, v, the output gate and the decays' low-rank logits side by side; with ``z = a2 low +
-    a2_bias`` (float32 ``[heads * dim, rank]`` and ``[heads * dim]``) a key channel's decay is
-    ``sigmoid(z)^(1/tau)``; ``S <- diag(decay) S + k v^T``, ``o = S^T (q_scale q)``.  ``state`` (float32
-    ``[slots, heads, dim, vdim]``) is read and left up to date.  Returns ``o / rms(o) * norm_weight *
-    silu(gate)`` as ``[tokens, heads * vdim]``."""
-    tokens = proj.shape[0]
+def _gla_checks(proj, state, a2, a2_bias, norm_weight, row_start, row_slots, rows, heads, dim, vdim, rank) -> None:
     q, v = heads * dim, heads * vdim
     if proj.dim() != 2 or proj.shape[1] != 2 * q + 2 * v + rank or proj.stride(1) != 1:
         raise KernelError("gla: the projection's rows must hold q, k, v, the gate and the decays' logits")
@@ -673,6 +664,20 @@ def gla_recurrent(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_
         raise KernelError(f"gla does not take heads of {dim} x {vdim}")
     if not proj.is_cuda:
         raise KernelError("proj must live on the GPU; there is no CPU path")
+
+
+def gla_recurrent(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_bias: torch.Tensor,
+                  norm_weight: torch.Tensor, row_start: torch.Tensor, row_slots: torch.Tensor, *, rows: int, heads: int,
+                  dim: int, vdim: int, rank: int, tau: float, eps: float, q_scale: float) -> torch.Tensor:
+    """Gated linear attention, token by token: ``proj`` ``[tokens, 2 heads dim + 2 heads vdim + rank]``
+    holds q, k, v, the output gate and the decays' low-rank logits side by side; with ``z = a2 low +
+    a2_bias`` (float32 ``[heads * dim, rank]`` and ``[heads * dim]``) a key channel's decay is
+    ``sigmoid(z)^(1/tau)``; ``S <- diag(decay) S + k v^T``, ``o = S^T (q_scale q)``.  ``state`` (float32
+    ``[slots, heads, dim, vdim]``) is read and left up to date.  Returns ``o / rms(o) * norm_weight *
+    silu(gate)`` as ``[tokens, heads * vdim]``."""
+    tokens = proj.shape[0]
+    q, v = heads * dim, heads * vdim
+    _gla_checks(proj, state, a2, a2_bias, norm_weight, row_start, row_slots, rows, heads, dim, vdim, rank)
     out = torch.empty((tokens, v), dtype=proj.dtype, device=proj.device)
     _lib.call("pylon_gla_recurrent", _dev(out, "out"), proj.data_ptr(), dtype_code(proj.dtype),
               proj.stride(0) if tokens > 1 else proj.shape[1], 0, q, 2 * q, 2 * q + v, 2 * q + 2 * v, rank,
@@ -683,13 +688,54 @@ def gla_recurrent(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_
     return out
 
 
+GLA_CHUNK = 64        # tokens of a chunk of gated linear attention with a workgroup of its own
+GLA_CHUNKED_FROM = 8  # a step whose longest row brings at least this many tokens takes the chunked form
+
+
+def gla_chunked_ok(dtype: torch.dtype, *, dim: int, vdim: int) -> bool:
+    """Whether the matrix-core form of gated linear attention takes this geometry (else the recurrent form)."""
+    return dtype == torch.bfloat16 and dim % 32 == 0 and 32 <= dim <= 256 and 1 <= vdim <= 256
+
+
+def gla_chunk_parallel(rows: int, heads: int, dim: int, vdim: int, max_count: int, units: Optional[int] = None) -> bool:
+    """Whether chunked gated linear attention takes one workgroup a chunk: when one workgroup a (row,
+    head) would leave most compute units idle, the rows are long enough for the two extra launches to
+    pay, and the chunks' states (float32, ``dim x vdim`` a chunk and head) fit a bound."""
+    units = units or _lib.compute_units()
+    chunks = -(-max_count // GLA_CHUNK)
+    return (rows * heads <= units and chunks >= 3
+            and rows * heads * chunks * dim * vdim * 4 <= RETENTION_PARALLEL_BYTES)
+
+
 def gla(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_bias: torch.Tensor, norm_weight: torch.Tensor,
         row_start: torch.Tensor, row_slots: torch.Tensor, *, rows: int, heads: int, dim: int, vdim: int, rank: int,
         tau: float, eps: float, q_scale: float, max_count: int) -> torch.Tensor:
     """Gated linear attention over the rows of a step (:func:`gla_recurrent` says what it computes);
-    ``max_count`` is the most tokens a row brings."""
-    return gla_recurrent(proj, state, a2, a2_bias, norm_weight, row_start, row_slots, rows=rows, heads=heads, dim=dim,
-                         vdim=vdim, rank=rank, tau=tau, eps=eps, q_scale=q_scale)
+    ``max_count`` is the most tokens a row brings.  Rows of a few tokens, float32 and odd sizes go token by
+    token; bfloat16 prompt portions sixteen tokens at a time on the matrix cores, with one workgroup a
+    (row, head), or, for few long rows, one a chunk of 64 tokens (:func:`gla_chunk_parallel`): what every
+    chunk adds to the state, a scan over the chunks, then every chunk's outputs."""
+    if max_count < GLA_CHUNKED_FROM or not gla_chunked_ok(proj.dtype, dim=dim, vdim=vdim):
+        return gla_recurrent(proj, state, a2, a2_bias, norm_weight, row_start, row_slots, rows=rows, heads=heads, dim=dim,
+                             vdim=vdim, rank=rank, tau=tau, eps=eps, q_scale=q_scale)
+    tokens = proj.shape[0]
+    q, v = heads * dim, heads * vdim
+    _gla_checks(proj, state, a2, a2_bias, norm_weight, row_start, row_slots, rows, heads, dim, vdim, rank)
+    out = torch.empty((tokens, v), dtype=proj.dtype, device=proj.device)
+    decays = torch.empty((tokens, q), dtype=torch.float32, device=proj.device)
+    chunk_state = chunk_log = None
+    if gla_chunk_parallel(rows, heads, dim, vdim, max_count):
+        chunks = rows * heads * -(-max_count // GLA_CHUNK)
+        chunk_state = torch.empty((chunks * dim * vdim,), dtype=torch.float32, device=proj.device)
+        chunk_log = torch.empty((chunks * dim,), dtype=torch.float32, device=proj.device)
+    _lib.call("pylon_gla_chunked", _dev(out, "out"), proj.data_ptr(), proj.stride(0) if tokens > 1 else proj.shape[1], 0, q,
+              2 * q, 2 * q + v, 2 * q + 2 * v, rank, _dev(a2, "a2", torch.float32), _dev(a2_bias, "a2_bias", torch.float32),
+              1.0 / float(tau), _dev(decays, "decays"), _dev(state, "state", torch.float32),
+              _dev(norm_weight, "norm_weight", torch.float32), _dev(row_start, "row_start", torch.int32),
+              _dev(row_slots, "row_slots", torch.int32), rows, heads, dim, vdim, float(eps), float(q_scale), int(max_count),
+              _dev(chunk_state, "chunk_state"), 0 if chunk_state is None else chunk_state.numel(),
+              _dev(chunk_log, "chunk_log"), 0 if chunk_log is None else chunk_log.numel(), _stream())
+    return out
 
 
 def kv_store(proj: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, slot_map: torch.Tensor, *,

@@ -154,7 +154,7 @@ def test_gated_linear_attention_in_portions_of_two_requests_over_reused_slots(op
     missed), or so strong that a channel is gone after a token or two."""
     rng = np.random.default_rng(heads * 1000 + dim + vdim)
     lengths = {"x": 201, "y": 23}
-    qk, vv, rank, tau = heads * dim, heads * vdim, 5, 3.0
+    qk, vv, rank, tau = heads * dim, heads * vdim, 8 if strong else 5, 3.0  # rows of the projection that are whole 16-byte pieces, or not
     data = {rid: {name: rounded(rng.normal(size=(n, size)), dtype) for name, size in
                   (("q", qk), ("k", qk), ("v", vv), ("gate", vv), ("low", rank))} for rid, n in lengths.items()}
     a2 = rng.normal(size=(qk, rank)).astype(np.float32).astype(np.float64) * (20.0 if strong else 1.0)
@@ -197,7 +197,7 @@ def test_gated_linear_attention_in_portions_of_two_requests_over_reused_slots(op
 def test_gated_linear_attention_over_many_and_long_rows(ops, rows, count, dtype):
     """However the kernel shares a step's rows and their pieces between workgroups."""
     rng = np.random.default_rng(rows)
-    heads, dim, vdim, rank, tau, eps = 2, 64, 48, 4, 6.0, 1e-6
+    heads, dim, vdim, rank, tau, eps = 2, 64, 48, 8, 6.0, 1e-6
     qk, vv = heads * dim, heads * vdim
     a2, bias = dev(rng.normal(size=(qk, rank))), dev(rng.normal(size=qk) + 3.0)
     norm_w = dev(1 + 0.2 * rng.normal(size=vdim))
