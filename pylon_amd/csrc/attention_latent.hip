@@ -380,7 +380,7 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(
     }
   }
 
-  // the waves' maxima and sums meet; a head's factor is that of its wave
+  // the waves' maxima and sums meet: per head the maximum of all, every wave's factor and the whole sum
 #pragma unroll
   for (int qt = 0; qt < QT; ++qt) {
     if (grp == 0) merge_m[wave][qt * 16 + col] = m_run[qt];
@@ -390,17 +390,36 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(
     }
   }
   __syncthreads();  // also: no wave reads its block any more
+  if (tid < HEADS) {
+    float m = merge_m[0][tid];
+#pragma unroll
+    for (int w = 1; w < 4; ++w) m = fmaxf(m, merge_m[w][tid]);
+    float l = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float mw = merge_m[w][tid];
+      const float fac = (mw == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f((mw - m) * scale_log2);
+      l = fmaf(merge_l[w][tid], fac, l);
+      merge_m[w][tid] = fac;
+    }
+    if (head0 + tid < n_heads) {
+      if (cuts > 1) {
+        float* dst = partial + ((static_cast<size_t>(tok) * n_heads + head0 + tid) * cuts + cut) * (2 + rank);
+        dst[0] = m * scale_log2;
+        dst[1] = l;
+      } else if (sink != nullptr) {
+        l += __builtin_amdgcn_exp2f(sink[head0 + tid] * AL_LOG2E - m * scale_log2);
+      }
+    }
+    merge_l[0][tid] = 1.0f / l;  // used where the keys are not cut
+  }
+  __syncthreads();
   float* stage = reinterpret_cast<float*>(al_lds);  // [4 waves][HEADS][16 CT]
 #pragma unroll
   for (int qt = 0; qt < QT; ++qt) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int h = qt * 16 + 4 * grp + r;
-      float m = merge_m[0][h];
-#pragma unroll
-      for (int w = 1; w < 4; ++w) m = fmaxf(m, merge_m[w][h]);
-      const float own = merge_m[wave][h];
-      const float fac = (own == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f((own - m) * scale_log2);
+      const float fac = merge_m[wave][qt * 16 + 4 * grp + r];
 #pragma unroll
       for (int nt = 0; nt < NT; ++nt) o[qt][nt][r] *= fac;
     }
@@ -416,56 +435,68 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(
         for (int r = 0; r < 4; ++r)
           stage[(wave * HEADS + qt * 16 + 4 * grp + r) * (16 * CT) + c * 16 + col] = o[qt][c0 + c][r];
     __syncthreads();
-    for (int i = tid; i < HEADS * 16 * CT; i += 256) {
+#pragma unroll
+    for (int j = 0; j < HEADS * 16 * CT / 1024; ++j) {  // four neighbouring elements a thread
+      const int i = (j * 256 + tid) * 4;
       const int h = i / (16 * CT), d = c0 * 16 + i % (16 * CT);
-      if (head0 + h >= n_heads || d >= rank) continue;
-      float m = merge_m[0][h];
+      float4 acc = *reinterpret_cast<const float4*>(stage + i);
 #pragma unroll
-      for (int w = 1; w < 4; ++w) m = fmaxf(m, merge_m[w][h]);
-      float acc = 0.f, l = 0.f;
-#pragma unroll
-      for (int w = 0; w < 4; ++w) {
-        acc += stage[w * HEADS * 16 * CT + i];
-        const float mw = merge_m[w][h];
-        l += (mw == -INFINITY) ? 0.f : merge_l[w][h] * __builtin_amdgcn_exp2f((mw - m) * scale_log2);
+      for (int w = 1; w < 4; ++w) {
+        const float4 x = *reinterpret_cast<const float4*>(stage + w * HEADS * 16 * CT + i);
+        acc.x += x.x; acc.y += x.y; acc.z += x.z; acc.w += x.w;
       }
+      if (head0 + h >= n_heads) continue;
+      const float v[4] = {acc.x, acc.y, acc.z, acc.w};
       const size_t item = static_cast<size_t>(tok) * n_heads + head0 + h;
-      if (cuts > 1) {
-        float* dst = partial + (item * cuts + cut) * (2 + rank);
-        if (d == 0) {
-          dst[0] = m * scale_log2;
-          dst[1] = l;
-        }
-        dst[2 + d] = acc;
-      } else {
-        if (sink != nullptr) l += __builtin_amdgcn_exp2f(sink[head0 + h] * AL_LOG2E - m * scale_log2);
-        out[item * rank + d] = float_to_bf16_bits(acc / l);
+      float* dst = partial + (item * cuts + cut) * (2 + rank) + 2 + d;
+      const float inv = merge_l[0][h];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        if (d + e >= rank) continue;
+        if (cuts > 1) dst[e] = v[e];
+        else out[item * rank + d + e] = float_to_bf16_bits(v[e] * inv);
       }
     }
   }
 }
 
-// One wave per (token, head) merges the cuts (at most 64) in their order; the sink joins here.
-__global__ void latent_merge_kernel(uint16_t* __restrict__ out, const float* __restrict__ partial, int items, int n_heads,
-                                    int cuts, int rank, const float* __restrict__ sink) {
-  const int item = blockIdx.x * (blockDim.x / PYLON_WAVE) + threadIdx.x / PYLON_WAVE;
+// One workgroup per (token, head) merges the cuts (at most 64) in their order; the sink joins here.  A
+// thread takes an element of the values; the loads of eight cuts do not wait for one another.
+__global__ __launch_bounds__(256) void latent_merge_kernel(uint16_t* __restrict__ out, const float* __restrict__ partial,
+                                                           int n_heads, int cuts, int rank, const float* __restrict__ sink) {
+  const int item = blockIdx.x;
   const int lane = threadIdx.x & (PYLON_WAVE - 1);
-  if (item >= items) return;
-  const float* src = partial + static_cast<size_t>(item) * cuts * (2 + rank);
-  const float mc = lane < cuts ? src[lane * (2 + rank)] : -INFINITY;
-  const float lc = lane < cuts ? src[lane * (2 + rank) + 1] : 0.f;
+  const int stride = 2 + rank;
+  const float* src = partial + static_cast<size_t>(item) * cuts * stride;
+  const float mc = lane < cuts ? src[lane * stride] : -INFINITY;
+  const float lc = lane < cuts ? src[lane * stride + 1] : 0.f;
+  const float z = sink != nullptr ? sink[item % n_heads] * AL_LOG2E : 0.f;
+  const int last = cuts - 1;
+  const int d0 = static_cast<int>(threadIdx.x) < rank ? static_cast<int>(threadIdx.x) : rank - 1;
+  float v[8];  // the first element's first cuts are on their way while the maxima meet
+#pragma unroll
+  for (int u = 0; u < 8; ++u) v[u] = src[(u < last ? u : last) * stride + 2 + d0];
   const float m = wave_max(mc);  // finite: some cut holds the token's own key
   const float w = (mc == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(mc - m);
   float l = wave_sum(lc * w);
-  if (sink != nullptr) l += __builtin_amdgcn_exp2f(sink[item % n_heads] * AL_LOG2E - m);
+  if (sink != nullptr) l += __builtin_amdgcn_exp2f(z - m);
   const float inv = 1.0f / l;
-  for (int d0 = 0; d0 < rank; d0 += PYLON_WAVE) {  // every lane stays in the loop: its weight is read by the others
-    const int d = d0 + lane;
-    const bool mine = d < rank;
+  for (int base = 0; base < rank; base += 256) {  // every lane stays in the loop: its weight is read by the others
+    const int d = base + threadIdx.x;
+    const int dd = d < rank ? d : rank - 1;
     float acc = 0.f;
-#pragma unroll 8
-    for (int c = 0; c < cuts; ++c) acc = fmaf(mine ? src[c * (2 + rank) + 2 + d] : 0.f, __shfl(w, c, PYLON_WAVE), acc);
-    if (mine) out[static_cast<size_t>(item) * rank + d] = float_to_bf16_bits(acc * inv);
+    for (int c0 = 0; c0 < cuts; c0 += 8) {
+      if (base != 0 || c0 != 0) {
+#pragma unroll
+        for (int u = 0; u < 8; ++u) v[u] = src[(c0 + u < last ? c0 + u : last) * stride + 2 + dd];
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const float f = __shfl(w, (c0 + u) & (PYLON_WAVE - 1), PYLON_WAVE);
+        if (c0 + u < cuts) acc = fmaf(v[u], f, acc);
+      }
+    }
+    if (d < rank) out[static_cast<size_t>(item) * rank + d] = float_to_bf16_bits(acc * inv);
   }
 }
 
@@ -568,8 +599,9 @@ extern "C" int pylon_latent_decode(void* out, const void* q, const void* cache, 
 #undef AL_GO
   if (cuts > 1) {
     const long long items = static_cast<long long>(tokens) * n_heads;
-    hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, stream, (uint16_t*)out,
-                       partial, static_cast<int>(items), n_heads, cuts, rank, sink);
+    PYLON_REQUIRE(items < (1ll << 31), "latent_decode: too many (token, head) pairs for one launch");
+    hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)items), dim3(256), 0, stream, (uint16_t*)out, partial, n_heads,
+                       cuts, rank, sink);
   }
   PYLON_LAUNCHED("latent_decode");
 }

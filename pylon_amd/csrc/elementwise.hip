@@ -655,6 +655,38 @@ __global__ void sigmoid_gate_kernel(T* __restrict__ x, const T* __restrict__ g, 
   }
 }
 
+// Eight bfloat16 elements (16 bytes) a thread; EACH: a gate per element (eight neighbours, 16 bytes as well), else
+// one for all eight (a head's size is a multiple of 8).
+template <bool EACH>
+__global__ void sigmoid_gate_bf16x8_kernel(uint4* __restrict__ x, const bf16_t* __restrict__ g, long long g_stride, int chunks,
+                                           int per, size_t total) {
+  size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
+  const size_t step = static_cast<size_t>(gridDim.x) * blockDim.x;
+  for (; i < total; i += step) {
+    const size_t t = i / chunks;
+    const int e = static_cast<int>(i - t * chunks) * 8;
+    const uint4 raw = x[i];
+    const uint32_t w[4] = {raw.x, raw.y, raw.z, raw.w};
+    uint32_t gw[4] = {0u, 0u, 0u, 0u};
+    float one = 0.f;
+    if constexpr (EACH) {
+      const uint4 graw = *reinterpret_cast<const uint4*>(g + t * g_stride + e);
+      gw[0] = graw.x; gw[1] = graw.y; gw[2] = graw.z; gw[3] = graw.w;
+    } else {
+      one = 1.0f / (1.0f + __expf(-to_float(g[t * g_stride + e / per])));
+    }
+    uint32_t r[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float ga = EACH ? 1.0f / (1.0f + __expf(-__uint_as_float(gw[j] << 16))) : one;
+      const float gb = EACH ? 1.0f / (1.0f + __expf(-__uint_as_float(gw[j] & 0xffff0000u))) : one;
+      const float a = __uint_as_float(w[j] << 16) * ga, b = __uint_as_float(w[j] & 0xffff0000u) * gb;
+      r[j] = static_cast<uint32_t>(float_to_bf16_bits(a)) | (static_cast<uint32_t>(float_to_bf16_bits(b)) << 16);
+    }
+    x[i] = uint4{r[0], r[1], r[2], r[3]};
+  }
+}
+
 // x: [rows, dim] of dtype, contiguous; g: [rows, dim / per] of the same dtype, rows g_stride apart.
 extern "C" int pylon_sigmoid_gate(void* x, int dtype, const void* g, long long g_stride, long long rows, int dim,
                                   int per, hipStream_t stream) {
@@ -663,6 +695,18 @@ extern "C" int pylon_sigmoid_gate(void* x, int dtype, const void* g, long long g
   PYLON_REQUIRE(g_stride >= dim / per, "sigmoid_gate: rows of gates overlap");
   const size_t total = static_cast<size_t>(rows) * dim;
   if (total == 0) return 0;
+  if (dtype == PYLON_BF16 && dim % 8 == 0 && (reinterpret_cast<uintptr_t>(x) & 15) == 0 &&
+      (per % 8 == 0 || (per == 1 && g_stride % 8 == 0 && (reinterpret_cast<uintptr_t>(g) & 15) == 0))) {
+    size_t wide = (total / 8 + 255) / 256;
+    if (wide > 65535u * 16u) wide = 65535u * 16u;
+    if (per == 1)
+      hipLaunchKernelGGL(sigmoid_gate_bf16x8_kernel<true>, dim3((unsigned)wide), dim3(256), 0, stream, (uint4*)x,
+                         (const bf16_t*)g, g_stride, dim / 8, per, total / 8);
+    else
+      hipLaunchKernelGGL(sigmoid_gate_bf16x8_kernel<false>, dim3((unsigned)wide), dim3(256), 0, stream, (uint4*)x,
+                         (const bf16_t*)g, g_stride, dim / 8, per, total / 8);
+    PYLON_LAUNCHED("sigmoid_gate");
+  }
   size_t blocks = (total + 255) / 256;
   if (blocks > 65535u * 16u) blocks = 65535u * 16u;
   if (dtype == PYLON_F32)

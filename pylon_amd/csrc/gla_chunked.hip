@@ -55,14 +55,14 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(float* __restrict__ b, c
                                                         int a_off, int rank, const float* __restrict__ a2,
                                                         const float* __restrict__ a2_bias, float inv_tau,
                                                         const int* __restrict__ row_start, int channels) {
-  extern __shared__ float low[];  // [GC_STEP][rank]
-  const int row = blockIdx.y;
+  extern __shared__ __attribute__((aligned(16))) float low[];  // [GC_STEP][rank rounded up to GD_RANK], zeros behind the rank
+  const int row = blockIdx.y, padded = (rank + GD_RANK - 1) / GD_RANK * GD_RANK;
   const int t0 = row_start[row] + blockIdx.x * GC_STEP, end = row_start[row + 1];
   if (t0 >= end) return;
   const int n = end - t0 < GC_STEP ? end - t0 : GC_STEP;
-  for (int i = threadIdx.x; i < GC_STEP * rank; i += 256) {
-    const int t = i / rank, r = i - t * rank;
-    low[i] = t < n ? to_float(proj[static_cast<size_t>(t0 + t) * ld + a_off + r]) : 0.f;
+  for (int i = threadIdx.x; i < GC_STEP * padded; i += 256) {
+    const int t = i / padded, r = i - t * padded;
+    low[i] = (t < n && r < rank) ? to_float(proj[static_cast<size_t>(t0 + t) * ld + a_off + r]) : 0.f;
   }
   __syncthreads();
   const int c = blockIdx.z * 256 + threadIdx.x;
@@ -78,8 +78,13 @@ __global__ __launch_bounds__(256) void gla_decay_kernel(float* __restrict__ b, c
 #pragma unroll
     for (int t = 0; t < GC_STEP; ++t)
 #pragma unroll
-      for (int r = 0; r < GD_RANK; ++r)
-        if (r0 + r < rank) z[t] = fmaf(low[t * rank + r0 + r], w[r], z[t]);
+      for (int r = 0; r < GD_RANK; r += 4) {
+        const float4 x = *reinterpret_cast<const float4*>(low + t * padded + r0 + r);
+        z[t] = fmaf(x.x, w[r], z[t]);
+        z[t] = fmaf(x.y, w[r + 1], z[t]);
+        z[t] = fmaf(x.z, w[r + 2], z[t]);
+        z[t] = fmaf(x.w, w[r + 3], z[t]);
+      }
   }
   const float bias = a2_bias[c];
   float sum = 0.f;
@@ -494,7 +499,7 @@ extern "C" int pylon_gla_chunked(void* out, const void* proj, long long ld, int 
   PYLON_REQUIRE(rows >= 0 && rows <= 65535 && heads > 0 && heads <= 65535 && max_count >= 1 && rank >= 1, "gla_chunked: bad sizes");
   PYLON_REQUIRE(dim >= 32 && dim % 32 == 0 && dim <= 256, "gla_chunked: keys of a multiple of 32 up to 256 elements, got %d", dim);
   PYLON_REQUIRE(vdim >= 1 && vdim <= 256, "gla_chunked: values of up to 256 elements, got %d", vdim);
-  PYLON_REQUIRE(rank <= 1024, "gla_chunked: at most 1024 logits of the decays, got %d", rank);
+  PYLON_REQUIRE(rank <= 512, "gla_chunked: at most 512 logits of the decays, got %d", rank);
   PYLON_REQUIRE((reinterpret_cast<uintptr_t>(proj) & 15) == 0 && (reinterpret_cast<uintptr_t>(b) & 15) == 0 && (reinterpret_cast<uintptr_t>(norm_w) & 15) == 0 &&
                     (reinterpret_cast<uintptr_t>(out) & 7) == 0, "gla_chunked: operands must be aligned");
   PYLON_REQUIRE(inv_tau > 0.f, "gla_chunked: tau must be positive");
@@ -506,7 +511,8 @@ extern "C" int pylon_gla_chunked(void* out, const void* proj, long long ld, int 
                 "gla_chunked: the chunks' states need rows x heads x chunks x dim x vdim floats, their decays x dim");
   const int channels = heads * dim;
   const int steps = (max_count + GC_STEP - 1) / GC_STEP;
-  hipLaunchKernelGGL(gla_decay_kernel, dim3(steps, rows, (channels + 255) / 256), dim3(256), sizeof(float) * GC_STEP * rank,
+  hipLaunchKernelGGL(gla_decay_kernel, dim3(steps, rows, (channels + 255) / 256), dim3(256),
+                     sizeof(float) * GC_STEP * ((rank + GD_RANK - 1) / GD_RANK * GD_RANK),
                      stream, b, (const bf16_t*)proj, ld, a_off, rank, a2, a2_bias, inv_tau, row_start, channels);
   const int nvw = vdim <= 64 ? 1 : vdim <= 128 ? 2 : 4;
   const size_t lds = 2 * (4 * static_cast<size_t>(GC_STEP) * (dim + 8) + static_cast<size_t>(GC_STEP) * (64 * nvw + 8)) +

@@ -12,6 +12,7 @@
 //   them, its four waves a quarter of n_in each; sums in float in one fixed order, whatever the batch.
 //   The heads of x and of out may lie apart (parts of wider heads), and the gate may come as raw logits
 //   of x's type, one per head or per element, whose sigmoid is taken here.
+// head_project_rows: the same for few bfloat16 tokens on the matrix cores, from a matrix that lies output by output.
 // gate_heads: x[t, h, :] *= gate[t, h] in place.
 //
 // Where a part of every key carries positions, the row of a token in the cache is [c | r]: the normed
@@ -223,15 +224,17 @@ head_project_kernel(TX* __restrict__ out, long long out_stride, int out_hstride,
 }
 
 // The same product for bfloat16 matrices whose rows are whole 16-byte pieces: a lane reads eight
-// neighbouring columns of a row of m[h] at once, sixteen lanes a 256-byte row segment, the sixteen
-// groups of lanes of a workgroup every sixteenth row; their sums meet by two shuffles inside a wave
-// and through LDS between the four waves, always in the same order.
-#define HW_COLS 128
+// neighbouring columns of a row of m[h] at once, the lanes of a row segment side by side, the groups of
+// lanes of a workgroup every 16th row; their sums meet by shuffles inside a
+// wave and through LDS between the four waves, always in the same order.
+#define HW_COLS 128  // outputs of a workgroup
 
 __global__ void __launch_bounds__(HP_THREADS)
 head_project_wide_kernel(bf16_t* __restrict__ out, long long out_stride, int out_hstride, const bf16_t* __restrict__ x,
                          long long x_stride, int x_hstride, const bf16_t* __restrict__ m, HeadGate<bf16_t> gate,
                          int tokens, int heads, int n_in, int n_out) {
+  constexpr int CG = HW_COLS / 8;              // lanes side by side on a row segment
+  constexpr int KG = HP_THREADS / CG;       // rows of m[h] under way at once
   extern __shared__ float xs[];  // [HP_TOKENS, n_in], then the waves' partial sums [4, HP_TOKENS, HW_COLS]
   float* partial = xs + HP_TOKENS * n_in;
   const int t0 = blockIdx.x * HP_TOKENS, h = blockIdx.y, c0 = blockIdx.z * HW_COLS, tid = threadIdx.x;
@@ -242,7 +245,7 @@ head_project_wide_kernel(bf16_t* __restrict__ out, long long out_stride, int out
   }
   __syncthreads();
   const int lane = tid & (PYLON_WAVE - 1), wave = tid / PYLON_WAVE;
-  const int cg = lane & 15, kg = wave * 4 + (lane >> 4);
+  const int cg = tid % CG, kg = tid / CG;
   float acc[HP_TOKENS][8];
 #pragma unroll
   for (int tt = 0; tt < HP_TOKENS; ++tt)
@@ -252,7 +255,7 @@ head_project_wide_kernel(bf16_t* __restrict__ out, long long out_stride, int out
   if (col < n_out) {  // n_out is a multiple of 8: the lane's eight columns are all inside
     const bf16_t* mh = m + static_cast<size_t>(h) * n_in * n_out + col;
 #pragma unroll 4
-    for (int k = kg; k < n_in; k += 16) {
+    for (int k = kg; k < n_in; k += KG) {
       const uint4 raw = *reinterpret_cast<const uint4*>(mh + static_cast<size_t>(k) * n_out);
       const uint32_t words[4] = {raw.x, raw.y, raw.z, raw.w};
       float wv[8];
@@ -274,9 +277,9 @@ head_project_wide_kernel(bf16_t* __restrict__ out, long long out_stride, int out
 #pragma unroll
     for (int c = 0; c < 8; ++c) {
       float v = acc[tt][c];
-      v += __shfl_xor(v, 16, PYLON_WAVE);
-      v += __shfl_xor(v, 32, PYLON_WAVE);
-      if (lane < 16) partial[(wave * HP_TOKENS + tt) * HW_COLS + 8 * cg + c] = v;
+#pragma unroll
+      for (int off = CG; off < PYLON_WAVE; off <<= 1) v += __shfl_xor(v, off, PYLON_WAVE);
+      if (lane < CG) partial[(wave * HP_TOKENS + tt) * HW_COLS + 8 * cg + c] = v;
     }
   __syncthreads();
   for (int i = tid; i < HP_TOKENS * HW_COLS; i += HP_THREADS) {
@@ -288,6 +291,101 @@ head_project_wide_kernel(bf16_t* __restrict__ out, long long out_stride, int out
     const float g = gate.at(t0 + tt, heads, h, n_out, c0 + c);
     out[static_cast<size_t>(t0 + tt) * out_stride + static_cast<size_t>(h) * out_hstride + c0 + c] = from_float<bf16_t>(sum * g);
   }
+}
+
+// The same product on the matrix cores for few tokens, from a matrix that lies output by output, mt[h] =
+// [n_out, n_in]: a wave owns 16 outputs of one head (the rows of the instruction) and all tokens (its
+// columns); every load of a few slabs of 32 inputs is sent for before the first product.  No LDS, no barrier;
+// the sums run along n_in in one order, whatever the batch.
+typedef __bf16 hp_bf16x8 __attribute__((ext_vector_type(8)));
+typedef float hp_floatx4 __attribute__((ext_vector_type(4)));
+typedef unsigned int hp_u32x4 __attribute__((ext_vector_type(4)));
+#define HM_SLABS 8  // slabs under way together
+#define HM_OUTPUTS 64  // outputs of a workgroup
+
+template <int TT>
+__global__ void __launch_bounds__(HP_THREADS)
+head_project_rows_kernel(bf16_t* __restrict__ out, long long out_stride, int out_hstride, const bf16_t* __restrict__ x,
+                         long long x_stride, int x_hstride, const bf16_t* __restrict__ mt, HeadGate<bf16_t> gate, int tokens,
+                         int heads, int n_in, int n_out) {
+  constexpr int SLABS = TT > 2 ? HM_SLABS / 2 : HM_SLABS;
+  const int lane = threadIdx.x & (PYLON_WAVE - 1), wave = threadIdx.x / PYLON_WAVE;
+  const int col = lane & 15, grp = lane >> 4;
+  const int h = blockIdx.x, o0 = blockIdx.y * HM_OUTPUTS + wave * 16;
+  if (o0 >= n_out) return;
+  const bf16_t* mrow = mt + (static_cast<size_t>(h) * n_out + (o0 + col < n_out ? o0 + col : n_out - 1)) * n_in;
+  const bf16_t* xrow[TT];
+  hp_floatx4 acc[TT];
+#pragma unroll
+  for (int t = 0; t < TT; ++t) {
+    const int tok = t * 16 + col;
+    xrow[t] = x + static_cast<size_t>(tok < tokens ? tok : tokens - 1) * x_stride + static_cast<size_t>(h) * x_hstride;
+    acc[t] = hp_floatx4{0.f, 0.f, 0.f, 0.f};
+  }
+  for (int k0 = 0; k0 < n_in; k0 += 32 * SLABS) {
+    hp_u32x4 a[SLABS], b[SLABS][TT];
+#pragma unroll
+    for (int s = 0; s < SLABS; ++s) {
+      const int k = k0 + s * 32 + grp * 8;
+      const bool in = k < n_in;  // n_in is a multiple of 8: the lane's eight inputs are all inside
+      a[s] = hp_u32x4{0u, 0u, 0u, 0u};
+      if (in) a[s] = *reinterpret_cast<const hp_u32x4*>(mrow + k);
+#pragma unroll
+      for (int t = 0; t < TT; ++t) {
+        b[s][t] = hp_u32x4{0u, 0u, 0u, 0u};
+        if (in) b[s][t] = *reinterpret_cast<const hp_u32x4*>(xrow[t] + k);
+      }
+    }
+#pragma unroll
+    for (int s = 0; s < SLABS; ++s)
+#pragma unroll
+      for (int t = 0; t < TT; ++t)
+        acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(hp_bf16x8, a[s]),
+                                                         __builtin_bit_cast(hp_bf16x8, b[s][t]), acc[t], 0, 0, 0);
+  }
+#pragma unroll
+  for (int t = 0; t < TT; ++t) {
+    const int tok = t * 16 + col;
+    if (tok >= tokens) continue;
+    bf16_t* dst = out + static_cast<size_t>(tok) * out_stride + static_cast<size_t>(h) * out_hstride;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int o = o0 + 4 * grp + i;
+      if (o < n_out) dst[o] = from_float<bf16_t>(acc[t][i] * gate.at(tok, heads, h, n_out, o));
+    }
+  }
+}
+
+// x, out and the gates as for pylon_head_project, at most 64 tokens; mt: bf16 [heads, n_out, n_in], n_in a
+// multiple of 8, mt and the rows of every head of x 16-byte aligned.
+extern "C" int pylon_head_project_rows(void* out, long long out_stride, int out_hstride, const void* x, long long x_stride,
+                                       int x_hstride, const void* mt, const float* gate, const void* gate_logits,
+                                       long long gate_stride, int gate_per, int tokens, int heads, int n_in, int n_out,
+                                       hipStream_t stream) {
+  PYLON_REQUIRE(tokens >= 0 && tokens <= 64 && heads > 0 && n_in > 0 && n_out > 0, "head_project_rows: bad sizes");
+  PYLON_REQUIRE(n_in % 8 == 0 && x_stride % 8 == 0 && x_hstride % 8 == 0 &&
+                    ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(mt)) & 15) == 0,
+                "head_project_rows: inputs must be whole 16-byte pieces");
+  PYLON_REQUIRE(x_hstride >= n_in && x_stride >= static_cast<long long>(heads - 1) * x_hstride + n_in,
+                "head_project_rows: rows of x overlap");
+  PYLON_REQUIRE(out_hstride >= n_out && out_stride >= static_cast<long long>(heads - 1) * out_hstride + n_out,
+                "head_project_rows: rows of the result overlap");
+  PYLON_REQUIRE(gate == nullptr || gate_logits == nullptr, "head_project_rows: gates or their logits, not both");
+  PYLON_REQUIRE(gate_logits == nullptr || (gate_per >= 1 && (static_cast<long long>(heads) * n_out) % gate_per == 0 &&
+                                           gate_stride >= static_cast<long long>(heads) * n_out / gate_per),
+                "head_project_rows: the gates' logits do not match the outputs");
+  if (tokens == 0) return 0;
+  const dim3 grid(heads, (n_out + HM_OUTPUTS - 1) / HM_OUTPUTS);
+  PYLON_REQUIRE(grid.y <= 65535, "head_project_rows: too many outputs per head for one launch");
+  const HeadGate<bf16_t> gates = {gate, (const bf16_t*)gate_logits, gate_stride, gate_per};
+#define GO(TT)                                                                                                      \
+  hipLaunchKernelGGL(head_project_rows_kernel<TT>, grid, dim3(HP_THREADS), 0, stream, (bf16_t*)out, out_stride,     \
+                     out_hstride, (const bf16_t*)x, x_stride, x_hstride, (const bf16_t*)mt, gates, tokens, heads, n_in, n_out)
+  if (tokens <= 16) GO(1);
+  else if (tokens <= 32) GO(2);
+  else GO(4);
+#undef GO
+  PYLON_LAUNCHED("head_project_rows");
 }
 
 // x: [tokens, heads, n_in], rows x_stride and heads x_hstride elements apart; m: [heads, n_in, n_out]; gate:

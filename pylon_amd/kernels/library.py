@@ -66,6 +66,7 @@ _SIGNATURES = {
     "pylon_latent_prefill": [P, P, P, P, I, P, I, I, I, I, I, I, F, P, I, P],
     "pylon_latent_decode": [P, P, P, P, I, P, I, I, I, I, I, I, F, P, I, P, L, P],
     "pylon_latent_rotate": [P, P, P, I, L, I, I, I, I, I, I, P, F, P, F, I, P, P, I, I, P],
+    "pylon_head_project_rows": [P, L, I, P, L, I, P, P, P, L, I, I, I, I, I, P],
     "pylon_head_project": [P, L, I, P, I, L, I, P, I, P, P, L, I, I, I, I, I, P],
     "pylon_gate_heads": [P, I, P, L, I, P],
     "pylon_route_top": [P, P, P, P, L, P, I, I, I, I, P],

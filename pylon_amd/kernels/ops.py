@@ -715,7 +715,7 @@ def gla(proj: torch.Tensor, state: torch.Tensor, a2: torch.Tensor, a2_bias: torc
     token; bfloat16 prompt portions sixteen tokens at a time on the matrix cores, with one workgroup a
     (row, head), or, for few long rows, one a chunk of 64 tokens (:func:`gla_chunk_parallel`): what every
     chunk adds to the state, a scan over the chunks, then every chunk's outputs."""
-    if max_count < GLA_CHUNKED_FROM or not gla_chunked_ok(proj.dtype, dim=dim, vdim=vdim):
+    if max_count < GLA_CHUNKED_FROM or rank > 512 or not gla_chunked_ok(proj.dtype, dim=dim, vdim=vdim):
         return gla_recurrent(proj, state, a2, a2_bias, norm_weight, row_start, row_slots, rows=rows, heads=heads, dim=dim,
                              vdim=vdim, rank=rank, tau=tau, eps=eps, q_scale=q_scale)
     tokens = proj.shape[0]
@@ -1229,14 +1229,17 @@ def _streaming_ok(x: torch.Tensor, weight: torch.Tensor, rows: int) -> bool:
 
 
 def gemm_skinny(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype = torch.bfloat16,
-                parts: int = 1, glu: bool = False,
+                parts: int = 1, glu: bool = False, relu2: bool = False,
                 out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``x @ weight.T`` for at most 64 rows of bfloat16 ``x``, streaming ``weight`` once.
 
     ``parts > 1`` cuts K into that many ranges and returns float32 partial results
     ``[parts, M, N]`` for the consumer to add.  ``glu``: ``weight`` is a fused
-    ``[2N, K]`` gate/up matrix and the result is ``silu(x @ gate.T) * (x @ up.T)``.
+    ``[2N, K]`` gate/up matrix and the result is ``silu(x @ gate.T) * (x @ up.T)``.  ``relu2``: the
+    result is ``max(x @ weight.T, 0)^2``.
     """
+    if relu2 and (glu or parts > 1):
+        raise KernelError("gemm_skinny: the squared relu takes the whole product, and no gate")
     if x.dim() != 2 or weight.dim() != 2 or x.shape[1] != weight.shape[1]:
         raise KernelError(f"gemm_skinny: cannot multiply {tuple(x.shape)} by the transpose of {tuple(weight.shape)}")
     m, k = x.shape
@@ -1256,12 +1259,12 @@ def gemm_skinny(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype
             or not out.is_cuda or not out.is_contiguous():
         raise KernelError(f"gemm_skinny: out must be contiguous, on the GPU and of shape {shape}")
     _lib.call("pylon_gemm_skinny", out.data_ptr(), dtype_code(out.dtype), x.data_ptr(), weight.data_ptr(),
-              m, n, k, x.stride(0), weight.stride(0), n, parts, m * n, 1 if glu else 0, _stream())
+              m, n, k, x.stride(0), weight.stride(0), n, parts, m * n, 2 if relu2 else (1 if glu else 0), _stream())
     return out
 
 
 def gemm_rows(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype = torch.bfloat16,
-              parts: int = 1, col_tiles: int = 1, glu: bool = False, waves: int = 0, cols: int = 0,
+              parts: int = 1, col_tiles: int = 1, glu: bool = False, relu2: bool = False, waves: int = 0, cols: int = 0,
               out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``x @ weight.T`` for at most 128 rows of bfloat16 ``x``: the rows of ``x`` pass through
     LDS once per workgroup of up to 64 (``col_tiles=1``) or 128 (``col_tiles=2``) columns and
@@ -1272,7 +1275,9 @@ def gemm_rows(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype =
     rounded once.  ``waves``: wavefronts per workgroup, 4 or 2 (0: the kernel's choice);
     ``cols``: columns per workgroup (0: the kernel's choice, an equal share for every
     workgroup of whole rounds over the compute units where that pays).  The sums depend on
-    neither."""
+    neither.  ``relu2``: the result is ``max(x @ weight.T, 0)^2``, rounded once."""
+    if relu2 and (glu or parts > 1):
+        raise KernelError("gemm_rows: the squared relu takes the whole product, and no gate")
     if x.dim() != 2 or weight.dim() != 2 or x.shape[1] != weight.shape[1]:
         raise KernelError(f"gemm_rows: cannot multiply {tuple(x.shape)} by the transpose of {tuple(weight.shape)}")
     m, k = x.shape
@@ -1292,7 +1297,7 @@ def gemm_rows(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype =
             or not out.is_cuda or not out.is_contiguous():
         raise KernelError(f"gemm_rows: out must be contiguous, on the GPU and of shape {shape}")
     _lib.call("pylon_gemm_rows", out.data_ptr(), dtype_code(out.dtype), x.data_ptr(), weight.data_ptr(),
-              m, n, k, x.stride(0), weight.stride(0), n, parts, m * n, int(col_tiles), 1 if glu else 0, int(waves),
+              m, n, k, x.stride(0), weight.stride(0), n, parts, m * n, int(col_tiles), 2 if relu2 else (1 if glu else 0), int(waves),
               int(cols), _stream())
     return out
 
@@ -1381,8 +1386,16 @@ def linear_glu(x: torch.Tensor, gate_up: torch.Tensor, *, out_dtype: torch.dtype
 
 
 def linear_relu2(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype) -> torch.Tensor:
-    """``max(x @ weight.T, 0)^2``.  Up to 128 rows the activation works on the product's float32 sums
-    and its result is rounded once; more bfloat16 rows: the library's product rounded first."""
+    """``max(x @ weight.T, 0)^2``.  Up to 128 bfloat16 rows the activation works on the product's float32
+    sums and its result is rounded once: in a streaming kernel's epilogue where one is the faster
+    product (:func:`plan.plan_projection`), else from the library's float32 result.  More rows: the
+    library's product rounded first."""
+    if _streaming_ok(x, weight, STREAM_ROWS):
+        choice = plan.plan_projection(x.shape[0], *weight.shape)
+        if choice.kernel == "rows":
+            return gemm_rows(x, weight, out_dtype=out_dtype, col_tiles=choice.col_tiles, relu2=True)
+        if choice.kernel == "skinny":
+            return gemm_skinny(x, weight, out_dtype=out_dtype, relu2=True)
     sums = torch.float32 if x.shape[0] <= SPLIT_ROWS else out_dtype
     return relu2(linear(x, weight, out_dtype=sums), out_dtype=out_dtype)
 
@@ -1676,12 +1689,14 @@ HEAD_PROJECT_ROWS = 64  # up to this many tokens the per-head products of bfloat
 
 
 def head_project(x: torch.Tensor, m: torch.Tensor, *, gate: Optional[torch.Tensor] = None,
-                 gate_logits: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                 gate_logits: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None,
+                 by_output: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``out[t, h] = gate[t, h] * x[t, h] @ m[h]`` for ``x`` ``[tokens, heads, n_in]`` and ``m`` ``[heads,
     n_in, n_out]``; ``gate`` float32 ``[tokens, heads]`` or None, or ``gate_logits`` of ``x``'s type
     ``[tokens, heads]`` or ``[tokens, heads * n_out]`` whose sigmoids multiply a head's outputs or every
     output.  ``x`` and ``out`` may be parts of wider heads and rows (``out`` is made if it is not given).
-    float32 operands and up to 64 bfloat16 tokens: the engine's kernel (float sums in the order of
+    ``by_output``: the same matrix output by output, ``[heads, n_out, n_in]``; with it up to 64 bfloat16
+    tokens of whole 16-byte pieces run on the matrix cores.  Otherwise float32 operands and up to 64 bfloat16 tokens: the engine's kernel (float sums in the order of
     ``n_in``, one rounding); more bfloat16 tokens: the library's batched product (where every size and
     distance is a multiple of 8 elements, or everything lies side by side), then the gate."""
     if x.dim() != 3 or m.dim() != 3 or m.shape[0] != x.shape[1] or m.shape[1] != x.shape[2]:
@@ -1703,6 +1718,18 @@ def head_project(x: torch.Tensor, m: torch.Tensor, *, gate: Optional[torch.Tenso
     elif out.shape != (tokens, heads, n_out) or out.dtype != x.dtype or not out.is_cuda or out.stride(2) != 1 \
             or out.stride(1) < n_out:
         raise KernelError("head_project: out must be [tokens, heads, n_out] of x's type with heads side by side")
+    logits_stride = 0 if gate_logits is None else (gate_logits.stride(0) if tokens > 1 else gate_logits.shape[1])
+    if by_output is not None and tokens <= HEAD_PROJECT_ROWS and x.dtype == torch.bfloat16 \
+            and by_output.dtype == torch.bfloat16 and n_in % 8 == 0 and x.stride(1) % 8 == 0 \
+            and (tokens == 1 or x.stride(0) % 8 == 0) and x.data_ptr() % 16 == 0:
+        if by_output.shape != (heads, n_out, n_in) or not by_output.is_contiguous() or by_output.data_ptr() % 16:
+            raise KernelError("head_project: by_output must be a contiguous [heads, n_out, n_in]")
+        _lib.call("pylon_head_project_rows", out.data_ptr(), out.stride(0) if tokens > 1 else heads * out.stride(1),
+                  out.stride(1), x.data_ptr(), x.stride(0) if tokens > 1 else heads * x.stride(1), x.stride(1),
+                  by_output.data_ptr(), _dev(gate, "gate", torch.float32),
+                  None if gate_logits is None else gate_logits.data_ptr(), logits_stride, per, tokens, heads, n_in, n_out,
+                  _stream())
+        return out
     together = x.stride(1) == n_in and out.is_contiguous()
     even = all(v % 8 == 0 for v in (n_in, n_out, x.stride(0), x.stride(1), out.stride(0), out.stride(1)))
     if x.dtype == torch.bfloat16 and m.dtype == torch.bfloat16 and tokens > HEAD_PROJECT_ROWS and (together or even):
@@ -1719,9 +1746,8 @@ def head_project(x: torch.Tensor, m: torch.Tensor, *, gate: Optional[torch.Tenso
     _lib.call("pylon_head_project", out.data_ptr(), out.stride(0) if tokens > 1 else heads * out.stride(1), out.stride(1),
               x.data_ptr(), dtype_code(x.dtype), x.stride(0) if tokens > 1 else heads * x.stride(1), x.stride(1),
               _dev(m, "m"), dtype_code(m.dtype), _dev(gate, "gate", torch.float32),
-              None if gate_logits is None else gate_logits.data_ptr(),
-              0 if gate_logits is None else (gate_logits.stride(0) if tokens > 1 else gate_logits.shape[1]), per, tokens,
-              heads, n_in, n_out, _stream())
+              None if gate_logits is None else gate_logits.data_ptr(), logits_stride, per, tokens, heads, n_in, n_out,
+              _stream())
     return out
 
 

@@ -83,21 +83,34 @@ class LatentAttention(Part):
             rotary = self.position.rotary()
             if rotary is not None and rotary[1] != spec.rot_dim:
                 raise ValueError(f"latent attention rotates its whole part of {spec.rot_dim} elements, not {rotary[1]}")
-        self._uv_by_latent = None  # (version of uv, uv as [heads, kv_rank, v_head_dim])
+        self._turned = {}  # parameter -> (its version, it with the last two axes of every head exchanged)
 
     def cache_requirement(self) -> KVRequirement:
         spec = self.spec
         return KVRequirement(1, self.width, spec.window, chunk=spec.chunk, values=False)
 
-    def value_maps(self) -> torch.Tensor:
-        """``uv`` with the latent's axis first inside every head, ``[heads, kv_rank, v_head_dim]``:
-        how the per-head product reads it; made anew when the parameter has been written."""
-        uv = self.params["uv"]
-        key = (uv.data_ptr(), uv._version, uv.dtype)
-        if self._uv_by_latent is None or self._uv_by_latent[0] != key:
-            spec = self.spec
-            self._uv_by_latent = (key, uv.view(spec.n_heads, spec.v_head_dim, spec.kv_rank).transpose(1, 2).contiguous())
-        return self._uv_by_latent[1]
+    def _map(self, name: str, rows: int) -> torch.Tensor:
+        """A per-head matrix as it is stored, ``[heads, rows, kv_rank]``."""
+        return self.params[name].view(self.spec.n_heads, rows, self.spec.kv_rank)
+
+    def _map_turned(self, name: str, rows: int) -> torch.Tensor:
+        """The same with the latent's axis first inside every head, ``[heads, kv_rank, rows]``; made anew
+        when the parameter has been written."""
+        param = self.params[name]
+        key = (param.data_ptr(), param._version, param.dtype)
+        if name not in self._turned or self._turned[name][0] != key:
+            self._turned[name] = (key, self._map(name, rows).transpose(1, 2).contiguous())
+        return self._turned[name][1]
+
+    def _into_latent(self, q: torch.Tensor, out=None) -> torch.Tensor:
+        """The queries' unrotated parts in the latent's space, ``q'_h = W_uk[h]^T q_h``."""
+        dim = self.spec.head_dim
+        return ops.head_project(q, self._map("uk", dim), out=out, by_output=self._map_turned("uk", dim))
+
+    def _into_values(self, mixed: torch.Tensor, **gating) -> torch.Tensor:
+        """Every head's weighted latent in its value space, ``W_uv[h] c``, times the gate."""
+        dim = self.spec.v_head_dim
+        return ops.head_project(mixed, self._map_turned("uv", dim), by_output=self._map("uv", dim), **gating)
 
     def _span(self, bound: int) -> int:
         limit = self.spec.window if self.spec.window is not None else self.spec.chunk
@@ -151,11 +164,9 @@ class LatentAttention(Part):
                 kv_rank=rank, n_gate=self.n_gate, q_weight=self.params["q_norm"], c_weight=self.params["c_norm"],
                 eps=spec.norm_eps, out_dtype=self.dtype)
             q = ops.linear(q_latent, self.params["uq"], out_dtype=self.dtype)
-            # the queries in the latent's space: q'_h = W_uk[h]^T q_h
-            q = ops.head_project(q.view(tokens, heads, spec.head_dim), self.params["uk"].view(heads, spec.head_dim, rank))
+            q = self._into_latent(q.view(tokens, heads, spec.head_dim))
         mixed = self._attend(q, ctx, cache)
-        # to the value space head by head, times the gate
-        context = ops.head_project(mixed, self.value_maps(), **gating)
+        context = self._into_values(mixed, **gating)
         return ops.linear_for_residual(context.view(tokens, heads * spec.v_head_dim), self.params["out"],
                                        out_dtype=self.dtype)
 
@@ -174,7 +185,7 @@ class LatentAttention(Part):
             rot_scale=self.position.rot_scale if rotary else 1.0,
             interleaved=self.position.interleaved if rotary else True, positions=ctx.positions)
         unrotated = proj[:, : self.q_rows].view(tokens, heads, spec.head_dim + spec.rot_dim)[..., : spec.head_dim]
-        ops.head_project(unrotated, self.params["uk"].view(heads, spec.head_dim, rank), out=q[..., :rank])
+        self._into_latent(unrotated, out=q[..., :rank])
         return q, proj[:, self.gate_off:] if self.n_gate else None
 
     def _attend(self, q: torch.Tensor, ctx, cache) -> torch.Tensor:

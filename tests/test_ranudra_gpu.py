@@ -275,7 +275,8 @@ def test_rows_and_queries_of_latent_attention(ops, heads, dim, rot, rank, vdim, 
                           interleaved=True, positions=i32(range(first, first + n)))
         q = proj[:, :q_size].reshape(n, heads, dim + rot)
         unrotated = moved[:, :q_size].view(n, heads, dim + rot)[..., :dim]
-        ops.head_project(unrotated, dev(uk, dtype), out=q_out[..., :rank])
+        ops.head_project(unrotated, dev(uk, dtype), out=q_out[..., :rank],
+                         by_output=dev(uk, dtype).transpose(1, 2).contiguous() if n == 9 else None)
         want_q = np.concatenate([np.einsum("thd,hdr->thr", q[..., :dim], uk), plain.rotate(q[..., dim:], raw, first)], axis=2)
         want_row = np.concatenate([plain.rms_norm(proj[:, q_size: q_size + rank], c_w, 1e-5),
                                    plain.rotate(proj[:, q_size + rank: q_size + rank + rot], raw, first)], axis=1)
@@ -305,6 +306,16 @@ def test_values_of_the_heads_with_gates_per_head_and_per_element(ops, heads, ran
         close(got.float().cpu().numpy(), plainly * plain.sigmoid(wide[:, 8: 8 + heads])[:, :, None], bound, "per head")
         got = ops.head_project(dev(x, dtype), dev(m, dtype), gate_logits=dev(wide, dtype)[:, 8:])
         close(got.float().cpu().numpy(), plainly * plain.sigmoid(wide[:, 8:]).reshape(plainly.shape), bound, "per element")
+        # with the matrix also output by output: the matrix cores where the sizes allow
+        turned = dev(m, dtype).transpose(1, 2).contiguous()
+        got = ops.head_project(dev(x, dtype), dev(m, dtype), gate_logits=dev(wide, dtype)[:, 8:], by_output=turned)
+        close(got.float().cpu().numpy(), plainly * plain.sigmoid(wide[:, 8:]).reshape(plainly.shape), bound, "by output")
+        gate = rng.uniform(size=(n, heads))
+        got = ops.head_project(dev(x, dtype), dev(m, dtype), gate=dev(gate), by_output=turned)
+        close(got.float().cpu().numpy(), plainly * gate[:, :, None], bound, "float gates")
+        if n > 1 and n <= 64:  # a token's result does not depend on its batch
+            one = ops.head_project(dev(x[-1:], dtype), dev(m, dtype), gate=dev(gate[-1:]), by_output=turned)
+            assert torch.equal(one[0], got[-1])
 
 
 def planted_rows(rng, n, heads, width, planted):
