@@ -1600,15 +1600,14 @@ def latent_attention_ok(dtype: torch.dtype, *, width: int, rank: int, page_size:
             and any(width <= w and rank <= r for w, r in _LATENT_SHAPES))
 
 
-def latent_rows(tokens: int, n_heads: int, rank: int) -> Optional[int]:
-    """Query rows of a workgroup of :func:`latent_prefill`: 128 halve the traffic from LDS per matrix
-    instruction, a step with few query rows fills more of the chip with workgroups of 64; values of more
-    than 256 elements leave registers for 64 only.  None: more heads than a workgroup takes."""
-    if rank > 256:
-        return 64 if n_heads <= 64 else None
-    if n_heads > 64:
-        return 128 if n_heads <= 128 else None
-    return 128 if tokens * n_heads >= 128 * 256 else 64
+def latent_rows(n_heads: int, rank: int) -> Optional[int]:
+    """Query rows of a workgroup of :func:`latent_prefill`: 64, two workgroups to a compute unit, unless the
+    heads are more (2,048 tokens, 32 heads, rows of 320 elements, a window of 1,024: 110 to 130 us against
+    162 with 128 rows, whose waves are alone on their SIMDs); values of more than 256 elements leave
+    registers for 64 only.  None: more heads than a workgroup takes."""
+    if n_heads <= 64:
+        return 64
+    return 128 if n_heads <= 128 and rank <= 256 else None
 
 
 def _latent_checks(name: str, q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor, rank: int,

@@ -218,7 +218,7 @@ class LatentAttention(Part):
                                          scale=spec.scale, rows=rows, out=mixed, **mask)
         if self._row_kernels(cache.page_size) and q.dtype == latents.dtype:
             options = dict(rank=rank, page_size=cache.page_size, scale=spec.scale, sink=self.params.get("sink"), **mask)
-            rows = ops.latent_rows(tokens, heads, rank)
+            rows = ops.latent_rows(heads, rank)
             # decoding requests at the head of a step go to the kernel of single tokens
             singles = tokens if ctx.decode_only else (ctx.leading_singles if rows else 0)
             if singles == tokens or rows:
