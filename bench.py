@@ -390,17 +390,17 @@ def ranudra_json(shape: dict, layers: int) -> dict:
     the middle stretch runs twice over the same weights (a quarter fewer layers own weights)."""
     width, hd, heads = shape["hidden_size"], shape["head_dim"], shape["num_attention_heads"]
     mlp = {"kind": "dense", "ff": shape["intermediate_size"] * 3 // 2}
-    linear = {"type": "gla", "mixer": {"heads": max(1, width // (2 * hd)), "dim": hd, "vdim": hd, "tau": 16.0}, "mlp": mlp}
+    linear = {"type": "gla", "mixer": {"heads": max(1, width // (2 * hd)), "dim": hd, "vdim": hd, "tau": 12.0}, "mlp": mlp}
     sizes = {"heads": heads, "dim": hd, "rot_dim": 64, "vdim": hd, "kv_rank": 256, "scale": (hd + 64) ** -0.5,
              "mask": {"size": 1024}}
     first = {"type": "latent_attention", "mlp": mlp, "mixer": {**sizes, "rot": {
-        "base": 1000000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
-    second = {"type": "latent_attention_2", "mlp": mlp, "mixer": {**sizes, "rot": {"base": 250000.0, "dims": 64}}}
+        "base": 500000.0, "dims": 64, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    second = {"type": "latent_attention_2", "mlp": mlp, "mixer": {**sizes, "rot": {"base": 100000.0, "dims": 64}}}
     again = layers // 4  # this many layers run twice
     own = layers - again
     start = (own - again) // 2
     return {"architecture": "Ranudra", "vocab": shape["vocab_size"], "width": width, "streams": 2,
-            "embedding": {"scale": 16.0}, "norm": {"eps": 1e-6},
+            "embedding": {"scale": 12.0}, "norm": {"eps": 1e-6},
             "loop": {"start": start, "stop": start + again, "times": 2} if again else None,
             "layers": [(linear, first, second)[i % 3] for i in range(own)]}
 

@@ -201,7 +201,7 @@ class LatentAttentionSpec:
 class GatedLinearAttentionSpec:
     """Linear attention with a learned, input-dependent decay per key channel: per request and head a
     float32 state ``S`` of ``head_dim x v_head_dim``, ``S_t = diag(alpha_t) S_(t-1) + k_t v_t^T``,
-    ``o_t = S_t^T q_t`` (the decay acts on the rows, which belong to key channels); ``q = W_q h *
+    ``o_t = S_t^T q_t`` (a row of ``S`` is a key channel's and fades by that channel's number); ``q = W_q h *
     head_dim ** -0.5``, ``alpha = sigmoid(W_a2 (W_a1 h) + b) ** (1 / tau)`` with ``decay_rank`` numbers
     between the two maps; every head's ``o`` is divided by its root mean square (``norm_eps`` inside the
     root), times a weight shared by the heads, times ``silu(W_g h)``; then the output projection."""
@@ -403,7 +403,8 @@ class LayerSpec:
 
     ``arrangement="hyper_connections"``: the residual stream is kept in ``streams`` copies ``x_1 .. x_s``
     (:attr:`ModelSpec.streams`), and every sublayer (mixer or feed-forward) has learned coefficients:
-    ``y = sublayer(norm(sum_s read[s] x_s))``, then, all copies at once, ``x_t <- sum_s mix[s, t] x_s +
+    ``y = sublayer(norm(sum_s read[s] x_s))``, after which every copy is renewed from what all of them held
+    before, ``x_t <- sum_s mix[s, t] x_s +
     write[t] y``.
     """
 

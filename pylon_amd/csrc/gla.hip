@@ -2,7 +2,7 @@
 // key channel.  Per request and head a state S [dim, vdim] of floats goes from token to token:
 //
 //   z = W_a2 (W_a1 h) + b,   alpha = sigmoid(z)^(1/tau)        (one number per key channel)
-//   S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t  (q times q_scale; the decay acts on S's rows)
+//   S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,   o_t = S_t^T q_t  (q times q_scale; a row of S belongs to a key channel)
 //   out_t = o_t / sqrt(mean(o_t^2) + eps) * w * silu(g_t)       (w: vdim numbers shared by the heads)
 //
 // The projection's rows hold q, k, v, g and the low-rank logits W_a1 h; W_a2 is applied here.

@@ -2,7 +2,7 @@
 // with the norm in front of the next sublayer:
 //
 //   d = sum_p delta[p]                              (the last sublayer's output, maybe as partial sums)
-//   x_t <- sum_s mix[s, t] x_s + write[t] d         (all copies at once, from the old ones)
+//   x_t <- sum_s mix[s, t] x_s + write[t] d         (each from what all copies held before)
 //   u = sum_t read[t] x_t                           (what the next sublayer, or the output, reads)
 //   out = (u - mean(u)) / sqrt(var(u) + eps) * w    (layer norm; without `centre` u / sqrt(mean(u^2) + eps) * w)
 //

@@ -113,7 +113,7 @@ def latent_mixer(h, m: dict, w: dict, pre: str, eps: float, *, gate: str) -> np.
 
 
 def gated_linear_attention(q, k, v, decay) -> np.ndarray:
-    """q, k, decay [n, H, dim], v [n, H, vdim] -> [n, H, vdim]: the decay acts on the state's rows."""
+    """q, k, decay [n, H, dim], v [n, H, vdim] -> [n, H, vdim]; row d of a head's state fades by decay[t, h, d]."""
     n, heads, dim = q.shape
     out = np.zeros_like(v)
     for h in range(heads):
@@ -149,8 +149,8 @@ def feed_forward(h, w: dict, pre: str) -> np.ndarray:
 
 
 def hyper_step(xs, sublayer, w: dict, pre: str) -> np.ndarray:
-    """xs [streams, n, width]: the sublayer reads one mix of the streams; every stream becomes a mix
-    of all the old ones plus its share of the sublayer's output."""
+    """xs [streams, n, width]: the sublayer reads a weighted sum of the streams; its output, weighted per
+    stream, joins a remix of what the streams held before."""
     u = np.einsum("s,snd->nd", w[pre + "in"], xs)
     y = sublayer(u)
     return np.einsum("st,snd->tnd", w[pre + "mix"], xs) + w[pre + "out"][:, None, None] * y

@@ -54,9 +54,9 @@ RANUDRA_A = _model(113, 40, 3, 5.0, 2e-5, [
 # B: rows that the matrix-core kernels take with room (80 of 96 and 128 elements), windows that are no
 # multiple of a page or a block, linear attention first and last, two copies, the loop at the end.
 RANUDRA_B = _model(160, 64, 2, 8.0, 1e-6, [
-    _layer("gla", _gla(2, 32, 64, 16.0), 88),
-    _layer("latent_attention", _latent(6, 32, 16, 48, 64, 0.17, _rot(1.0e6, 16, (8.0, 64, 16.0, 2.0)), 50), 72),
-    _layer("latent_attention_2", _latent(8, 16, 32, 24, 96, 0.2, _rot(2.5e5, 32), 100), 96),
+    _layer("gla", _gla(2, 32, 64, 10.0), 88),
+    _layer("latent_attention", _latent(6, 32, 16, 48, 64, 0.17, _rot(8.0e5, 16, (6.0, 64, 16.0, 2.0)), 50), 72),
+    _layer("latent_attention_2", _latent(8, 16, 32, 24, 96, 0.2, _rot(3.0e5, 32), 100), 96),
     _layer("gla", _gla(4, 16, 32, 9.0, 8), 64),
 ], (2, 4, 3))
 # C: more than 16 heads, a row of 256 + 64 elements and one of 128 + 32 that sees every earlier key, four
@@ -75,7 +75,7 @@ RANUDRA_D = _model(203, 96, 1, 11.0, 1e-5, [
     _layer("gla", _gla(1, 256, 24, 20.0, 2), 160),
 ])
 # E: a width of 100, a vocabulary of 301, the widest rows (512 + 64), strong decays (tau 0.5).
-RANUDRA_E = _model(301, 100, 2, 16.0, 1e-6, [
+RANUDRA_E = _model(301, 100, 2, 14.0, 1e-6, [
     _layer("latent_attention_2", _latent(2, 20, 64, 12, 512, 0.1, _rot(1.0e4, 64), 90), 60),
     _layer("gla", _gla(3, 32, 48, 0.5, 4), 44),
     _layer("latent_attention", _latent(3, 12, 4, 10, 28, 0.3, _rot(777.0, 4, (3.0, 20, 5.0, 1.0)), 9), 52),

@@ -141,7 +141,7 @@ def plain_gla_outputs(q, k, v, gate, low, a2, bias, norm_w, heads, dim, vdim, ta
     return plain.rms_norm(o, norm_w, eps).reshape(n, -1) * plain.silu(gate)
 
 
-GLA_SHAPES = [(4, 32, 32), (2, 12, 20), (3, 64, 128), (2, 128, 128), (1, 256, 64), (2, 128, 32), (1, 100, 24), (5, 1, 1),
+GLA_SHAPES = [(3, 32, 32), (2, 12, 20), (3, 64, 128), (2, 128, 128), (1, 256, 64), (2, 128, 32), (1, 100, 24), (5, 1, 1),
               (2, 48, 200), (1, 32, 256), (1, 64, 16), (2, 96, 80)]
 
 
@@ -248,8 +248,8 @@ def test_gated_linear_attention_keeps_what_it_wrote_far_back(ops, dtype):
 # ---- latent attention ----------------------------------------------------------------------------------
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("heads, dim, rot, rank, vdim, scaled", [(3, 10, 6, 18, 14, True), (6, 32, 32, 64, 32, True),
-                                                                  (8, 16, 64, 128, 80, False), (1, 8, 2, 8, 4, False)])
+@pytest.mark.parametrize("heads, dim, rot, rank, vdim, scaled", [(3, 10, 6, 18, 14, True), (6, 24, 32, 64, 40, True),
+                                                                  (7, 16, 64, 120, 72, False), (1, 8, 2, 8, 4, False)])
 def test_rows_and_queries_of_latent_attention(ops, heads, dim, rot, rank, vdim, scaled, dtype):
     """The latent normed and the shared key part rotated into scattered slots, the queries' rotated
     parts turned and their other parts carried into the latent's space (few tokens and many)."""
@@ -295,7 +295,7 @@ def test_rows_and_queries_of_latent_attention(ops, heads, dim, rot, rank, vdim, 
 
 
 @pytest.mark.parametrize("n", [1, 7, 64, 65, 200])
-@pytest.mark.parametrize("heads, rank, vdim", [(3, 18, 14), (6, 64, 32), (8, 128, 80), (2, 512, 16)])
+@pytest.mark.parametrize("heads, rank, vdim", [(3, 18, 14), (5, 64, 32), (8, 136, 80), (2, 512, 16)])
 def test_values_of_the_heads_with_gates_per_head_and_per_element(ops, heads, rank, vdim, n):
     rng = np.random.default_rng(n + rank)
     for dtype, bound in ((torch.float32, 2e-5), (torch.bfloat16, 1.5e-2)):
@@ -333,7 +333,7 @@ def planted_rows(rng, n, heads, width, planted):
 @pytest.mark.parametrize("size", [37, 64, 129, 1, 300, None])
 @pytest.mark.parametrize("dtype, heads, width, rank, page", [
     (torch.float32, 3, 28, 18, 16), (torch.float32, 2, 96, 64, 64), (torch.float32, 2, 576, 512, 64),
-    (torch.bfloat16, 6, 96, 64, 64), (torch.bfloat16, 8, 160, 128, 64), (torch.bfloat16, 3, 56, 40, 128),
+    (torch.bfloat16, 7, 96, 64, 64), (torch.bfloat16, 9, 160, 112, 64), (torch.bfloat16, 3, 56, 40, 128),
     (torch.bfloat16, 17, 128, 96, 64), (torch.bfloat16, 32, 320, 256, 256), (torch.bfloat16, 40, 192, 128, 64),
     (torch.bfloat16, 5, 256, 104, 64), (torch.bfloat16, 16, 384, 248, 64), (torch.bfloat16, 4, 576, 512, 64),
     (torch.bfloat16, 20, 576, 512, 64), (torch.bfloat16, 100, 72, 64, 64), (torch.bfloat16, 1, 8, 8, 64)])
