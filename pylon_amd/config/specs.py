@@ -43,13 +43,26 @@ class RotaryScalingSpec:
 
 
 @dataclass(frozen=True)
+class RotaryBandScalingSpec:
+    """Another way to stretch frequencies, by wavelength: with ``l = 2 pi / f``, a pair keeps its
+    frequency where ``l < original / high``, turns at ``f / factor`` where ``l > original / low``, and
+    between the two at ``(1 - s) f / factor + s f`` with ``s = (original / l - low) / (high - low)``.
+    Cosines and sines stay as they are."""
+
+    factor: float
+    low: float
+    high: float
+    original: float
+
+
+@dataclass(frozen=True)
 class PositionSpec:
     """How positions enter a mixer.
 
     ``kind="rope"``: rotate the first ``rotary_dim`` elements of every head by
     ``position * theta**(-2i/rotary_dim)``, pairing element ``i`` with
     ``i + rotary_dim/2``.  ``kind="none"``: positions are not encoded.
-    ``scaling``: see :class:`RotaryScalingSpec`.
+    ``scaling``: see :class:`RotaryScalingSpec` and :class:`RotaryBandScalingSpec`.
     """
 
     kind: str
@@ -58,7 +71,7 @@ class PositionSpec:
     max_positions: int = 0
     # True: element 2i turns together with its neighbour 2i + 1 instead of with i + rotary_dim/2
     interleaved: bool = False
-    scaling: Optional[RotaryScalingSpec] = None
+    scaling: Optional[object] = None
 
 
 @dataclass(frozen=True)
@@ -235,6 +248,23 @@ class RetentionSpec:
 
 
 @dataclass(frozen=True)
+class LightningAttentionSpec:
+    """Linear attention with one fixed decay per head on activated projections: ``q = silu(W_q h)``,
+    ``k = silu(W_k h)``, ``v = silu(W_v h)``, per request and head a float32 state
+    ``S_t = decay_h S_{t-1} + k_t v_t^T``, ``o_t = S_t^T q_t``; the concatenated heads are divided by their
+    common root mean square (``norm_eps`` inside the root), multiplied by a weight and by
+    ``sigmoid(W_g h)``, and projected."""
+
+    hidden_size: int
+    n_heads: int
+    head_dim: int
+    v_head_dim: int
+    decay: Tuple[float, ...]
+    norm_eps: float
+    kind: str = "lightning_attention"
+
+
+@dataclass(frozen=True)
 class DeltaRuleSpec:
     """The gated delta rule: per request and head a float32 state ``S`` of ``head_dim x v_head_dim``,
     ``S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q`` (the read-out sees the token's own
@@ -328,7 +358,9 @@ class MixtureFeedForwardSpec:
     output is the input itself.
 
     ``scoring="sigmoid"``: the scores are the sigmoids of the router's outputs, the ``top`` largest
-    are chosen and their scores are the weights as they are.  ``weight_on_input``: a chosen expert's
+    are chosen and their scores are the weights as they are; groups as above; ``group_score="top2"``: a
+    group counts with the sum of its two largest scores instead of its largest; ``renormalize``: the
+    weights are the chosen scores divided by their sum (+ 1e-20).  ``weight_on_input``: a chosen expert's
     weight multiplies its input instead of its output, ``sum_e expert_e(w_e h)``."""
 
     hidden_size: int
@@ -346,6 +378,8 @@ class MixtureFeedForwardSpec:
     groups_kept: int = 1
     route_scale: float = 1.0
     weight_on_input: bool = False
+    group_score: str = "max"
+    renormalize: bool = False
 
 
 @dataclass(frozen=True)
@@ -366,8 +400,8 @@ class LogitScaleSpec:
 
 @dataclass(frozen=True)
 class GatedFeedForwardSpec:
-    """``down(act(gate(x)) * up(x))`` with gate and up fused into one matrix; with ``bias`` all
-    three projections have one."""
+    """``down(act(gate(x)) * up(x))`` with gate and up fused into one matrix; ``activation``: "silu" or
+    "gelu_tanh" (gelu's tanh form); with ``bias`` (silu only) all three projections have one."""
 
     hidden_size: int
     intermediate_size: int
@@ -399,7 +433,8 @@ class LayerSpec:
     ``norm1``'s output; with ``sublayer_scale`` each sublayer's output is multiplied element by element
     by a learned vector before it is added; ``depth_mix = (index, total)`` makes the layer's result
     stream ``index`` of ``total`` (stream 0: the embedded tokens) and hands on, instead of it, a learned
-    mix ``sum_{j <= index} c[j] * stream_j`` of all streams so far.
+    mix ``sum_{j <= index} c[j] * stream_j`` of all streams so far; ``residual_factor`` multiplies both
+    sublayers' outputs as they are added.
 
     ``arrangement="hyper_connections"``: the residual stream is kept in ``streams`` copies ``x_1 .. x_s``
     (:attr:`ModelSpec.streams`), and every sublayer (mixer or feed-forward) has learned coefficients:
@@ -419,10 +454,22 @@ class LayerSpec:
     sublayer_scale: bool = False
     depth_mix: Optional[Tuple[int, int]] = None
     streams: int = 1
+    residual_factor: float = 1.0
 
     @property
     def kind(self) -> str:
         return self.arrangement
+
+
+@dataclass(frozen=True)
+class PassEntrySpec:
+    """What happens to the residual stream ahead of a pass through layers that run several times:
+    ``x <- W [x; x0] + step[t]``, with ``x0`` the embedded tokens, ``W`` one matrix for all passes and
+    ``step[t]`` a learned vector of pass ``t`` of ``times``."""
+
+    dim: int
+    times: int
+    kind: str = "join_embedding"
 
 
 @dataclass(frozen=True)
@@ -441,6 +488,9 @@ class ScheduleEntry:
     # True: the embedded tokens (the stream as it was before the first run) are added to the
     # stream once more right before this run
     add_embedding: bool = False
+    # t: pass number t through a stretch of layers begins right before this run, and the model's
+    # `pass_entry` part changes the stream there
+    begins_pass: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -461,6 +511,8 @@ class ModelSpec:
     # copies of the residual stream that the layers work on (all equal to the embedded tokens at first;
     # the final norm reads their sum)
     streams: int = 1
+    # the part (family "pass") that changes the stream before the runs that begin a pass
+    pass_entry: Optional[object] = None
     extra: dict = field(default_factory=dict, compare=False, hash=False)
 
     def resolved_schedule(self) -> Tuple[Tuple[int, int, bool], ...]:

@@ -45,6 +45,18 @@ __device__ __forceinline__ bf16_t from_float<bf16_t>(float v) {
   return r;
 }
 
+// The activations of gated feed-forwards.  gelu is its tanh form, 0.5 z (1 + tanh(c (z + 0.044715 z^3)))
+// with c = sqrt(2 / pi); because (1 + tanh(u)) / 2 = 1 / (1 + exp(-2u)) it costs one exponential.
+#define PYLON_ACT_SILU 0
+#define PYLON_ACT_GELU 1
+__device__ __forceinline__ float pylon_silu(float z) { return z / (1.0f + expf(-z)); }
+__device__ __forceinline__ float pylon_gelu_tanh(float z) {
+  return z / (1.0f + expf(-1.5957691216057308f * fmaf(0.044715f * z * z, z, z)));
+}
+__device__ __forceinline__ float pylon_gate_act(float z, int act) {
+  return act == PYLON_ACT_GELU ? pylon_gelu_tanh(z) : pylon_silu(z);
+}
+
 // Sum / max over the 64 lanes of a wavefront; every lane gets the result.
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

@@ -67,7 +67,7 @@ __device__ __forceinline__ void store4(bf16_t* p, long long c, float a, float b,
 // ---- RMSNorm ----------------------------------------------------------------------
 // y = (x * 1/sqrt(mean(x^2) + eps)) * w, in float, rounded once on the store.
 // One workgroup per output row. `row_idx` (optional) picks the input row of each
-// output row. With `delta`, the input is resid + delta (float sum); `write_resid`
+// output row. With `delta`, the input is resid + factor * delta (float sum); `write_resid`
 // stores that sum back into resid (only meaningful without row_idx).
 // At most 512 threads per workgroup, so that a thread may hold the eight partial sums of its
 // sixteen elements in registers (a kernel that may be launched with 1,024 threads gets 128).
@@ -75,7 +75,7 @@ template <typename TX, typename TD, typename TO>
 __global__ __launch_bounds__(512) void rmsnorm_kernel(TO* __restrict__ out, TX* x, const TD* __restrict__ delta,
                                int n_delta, long long delta_stride,
                                const float* __restrict__ w, const int* __restrict__ row_idx,
-                               int dim, float eps, int write_resid) {
+                               int dim, float eps, int write_resid, float factor) {
   __shared__ float scratch[16];
   const int r_out = blockIdx.x;
   const int r_in = row_idx ? row_idx[r_out] : r_out;
@@ -143,7 +143,10 @@ __global__ __launch_bounds__(512) void rmsnorm_kernel(TO* __restrict__ out, TX* 
 #undef PYLON_SUM_PARTS
 #pragma unroll
       for (int n = 0; n < VEC; ++n) {
-        held[n].x += d[n].x; held[n].y += d[n].y; held[n].z += d[n].z; held[n].w += d[n].w;
+        held[n].x = fmaf(factor, d[n].x, held[n].x);
+        held[n].y = fmaf(factor, d[n].y, held[n].y);
+        held[n].z = fmaf(factor, d[n].z, held[n].z);
+        held[n].w = fmaf(factor, d[n].w, held[n].w);
       }
     }
     float ss = 0.f;
@@ -171,7 +174,7 @@ __global__ __launch_bounds__(512) void rmsnorm_kernel(TO* __restrict__ out, TX* 
     if (dr) {
       float d = to_float(dr[i]);
       for (int p = 1; p < n_delta; ++p) d += to_float(dr[i + p * delta_stride]);
-      v += d;
+      v = fmaf(factor, d, v);
       if (write_resid) xr[i] = from_float<TX>(v);
     }
     ss += v * v;
@@ -183,7 +186,7 @@ __global__ __launch_bounds__(512) void rmsnorm_kernel(TO* __restrict__ out, TX* 
     if (dr && !write_resid) {
       float d = to_float(dr[i]);
       for (int p = 1; p < n_delta; ++p) d += to_float(dr[i + p * delta_stride]);
-      v += d;
+      v = fmaf(factor, d, v);
     }
     yr[i] = from_float<TO>((v * inv) * w[i]);
   }
@@ -200,7 +203,7 @@ template <typename TD, typename TO, int R, int THREADS>
 __global__ __launch_bounds__(THREADS) void add_rmsnorm_many_kernel(TO* __restrict__ out, float* resid,
                                                                const TD* __restrict__ delta,
                                                                const float* __restrict__ w, int rows, int dim,
-                                                               float eps) {
+                                                               float eps, float factor) {
   __shared__ float scratch[16];
   constexpr int VEC = 4;
   const int chunks = dim >> 2;
@@ -223,7 +226,7 @@ __global__ __launch_bounds__(THREADS) void add_rmsnorm_many_kernel(TO* __restric
       if (c < chunks) {
         const float4 x = reinterpret_cast<const float4*>(xr)[c];
         const float4 d = load4(dr, c);
-        held[i][n] = float4{x.x + d.x, x.y + d.y, x.z + d.z, x.w + d.w};
+        held[i][n] = float4{fmaf(factor, d.x, x.x), fmaf(factor, d.y, x.y), fmaf(factor, d.z, x.z), fmaf(factor, d.w, x.w)};
       } else {
         held[i][n] = float4{0.f, 0.f, 0.f, 0.f};
       }
@@ -258,7 +261,7 @@ __global__ __launch_bounds__(THREADS) void add_rmsnorm_many_kernel(TO* __restric
 template <typename TX, typename TD>
 static void launch_rmsnorm_out(void* out, int out_dtype, TX* x, const TD* delta, int n_delta,
                                long long delta_stride, const float* w, const int* row_idx, int rows,
-                               int dim, float eps, int write_resid, hipStream_t stream) {
+                               int dim, float eps, int write_resid, float factor, hipStream_t stream) {
   if constexpr (sizeof(TX) == 4) {
     if (rows >= PYLON_NORM_MANY_ROWS && delta != nullptr && n_delta == 1 && row_idx == nullptr && write_resid &&
         (dim & 3) == 0 && dim <= 8192) {
@@ -266,7 +269,7 @@ static void launch_rmsnorm_out(void* out, int out_dtype, TX* x, const TD* delta,
       dim3 grid((rows + R - 1) / R);
 #define GO(TO, THREADS)                                                                                    \
   hipLaunchKernelGGL((add_rmsnorm_many_kernel<TD, TO, R, THREADS>), grid, dim3(THREADS), 0, stream, (TO*)out, x, \
-                     delta, w, rows, dim, eps)
+                     delta, w, rows, dim, eps, factor)
       if (dim > 4096) {
         if (out_dtype == PYLON_F32) GO(float, 512); else GO(bf16_t, 512);
       } else {
@@ -279,10 +282,10 @@ static void launch_rmsnorm_out(void* out, int out_dtype, TX* x, const TD* delta,
   dim3 grid(rows), block(dim > 4096 ? 512 : 256);
   if (out_dtype == PYLON_F32)
     hipLaunchKernelGGL((rmsnorm_kernel<TX, TD, float>), grid, block, 0, stream, (float*)out, x, delta,
-                       n_delta, delta_stride, w, row_idx, dim, eps, write_resid);
+                       n_delta, delta_stride, w, row_idx, dim, eps, write_resid, factor);
   else
     hipLaunchKernelGGL((rmsnorm_kernel<TX, TD, bf16_t>), grid, block, 0, stream, (bf16_t*)out, x,
-                       delta, n_delta, delta_stride, w, row_idx, dim, eps, write_resid);
+                       delta, n_delta, delta_stride, w, row_idx, dim, eps, write_resid, factor);
 }
 
 // out[r] = rmsnorm(x[idx(r)]) for any input dtype.
@@ -294,19 +297,20 @@ extern "C" int pylon_rmsnorm(void* out, int out_dtype, const void* x, int x_dtyp
   if (rows == 0) return 0;
   if (x_dtype == PYLON_F32)
     launch_rmsnorm_out<float, float>(out, out_dtype, (float*)x, nullptr, 0, 0, w, row_idx, rows, dim,
-                                     eps, 0, stream);
+                                     eps, 0, 1.0f, stream);
   else
     launch_rmsnorm_out<bf16_t, bf16_t>(out, out_dtype, (bf16_t*)x, nullptr, 0, 0, w, row_idx, rows, dim,
-                                       eps, 0, stream);
+                                       eps, 0, 1.0f, stream);
   PYLON_LAUNCHED("rmsnorm");
 }
 
-// resid (float) += delta, then out = rmsnorm(resid). With row_idx the sum is formed only
+// resid (float) += factor * delta, then out = rmsnorm(resid). With row_idx the sum is formed only
 // for the picked rows and resid is left untouched. delta may come as n_delta partial sums,
 // delta_stride elements apart, which are added up first.
 extern "C" int pylon_add_rmsnorm(void* out, int out_dtype, float* resid, const void* delta,
                                  int delta_dtype, int n_delta, long long delta_stride, const float* w,
-                                 const int* row_idx, int rows, int dim, float eps, hipStream_t stream) {
+                                 const int* row_idx, int rows, int dim, float eps, float factor,
+                                 hipStream_t stream) {
   PYLON_REQUIRE(pylon_valid_dtype(out_dtype), "add_rmsnorm: unknown out dtype");
   PYLON_REQUIRE(delta == nullptr || pylon_valid_dtype(delta_dtype), "add_rmsnorm: unknown delta dtype");
   PYLON_REQUIRE(rows >= 0 && dim > 0, "add_rmsnorm: bad sizes rows=%d dim=%d", rows, dim);
@@ -315,10 +319,10 @@ extern "C" int pylon_add_rmsnorm(void* out, int out_dtype, float* resid, const v
   const int write_resid = (delta != nullptr && row_idx == nullptr) ? 1 : 0;
   if (delta == nullptr || delta_dtype == PYLON_F32)
     launch_rmsnorm_out<float, float>(out, out_dtype, resid, (const float*)delta, n_delta, delta_stride,
-                                     w, row_idx, rows, dim, eps, write_resid, stream);
+                                     w, row_idx, rows, dim, eps, write_resid, factor, stream);
   else
     launch_rmsnorm_out<float, bf16_t>(out, out_dtype, resid, (const bf16_t*)delta, n_delta,
-                                      delta_stride, w, row_idx, rows, dim, eps, write_resid, stream);
+                                      delta_stride, w, row_idx, rows, dim, eps, write_resid, factor, stream);
   PYLON_LAUNCHED("add_rmsnorm");
 }
 
@@ -347,9 +351,9 @@ extern "C" int pylon_residual_add(float* resid, const void* delta, int delta_dty
 }
 
 // ---- gated activation -----------------------------------------------------------------
-// out[t, i] = silu(gu[t, i]) * gu[t, inter + i]; silu(z) = z / (1 + exp(-z)).
+// out[t, i] = act(gu[t, i]) * gu[t, inter + i]; act: silu(z) = z / (1 + exp(-z)), or gelu's tanh form.
 template <typename TI, typename TO>
-__global__ void silu_gate_kernel(TO* __restrict__ out, const TI* __restrict__ gu, int inter, size_t total) {
+__global__ void silu_gate_kernel(TO* __restrict__ out, const TI* __restrict__ gu, int inter, size_t total, int act) {
   size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   const size_t step = static_cast<size_t>(gridDim.x) * blockDim.x;
   for (; i < total; i += step) {
@@ -357,14 +361,13 @@ __global__ void silu_gate_kernel(TO* __restrict__ out, const TI* __restrict__ gu
     const size_t c = i - t * inter;
     const float g = to_float(gu[t * 2 * inter + c]);
     const float u = to_float(gu[t * 2 * inter + inter + c]);
-    const float s = g / (1.0f + expf(-g));
-    out[i] = from_float<TO>(s * u);
+    out[i] = from_float<TO>(pylon_gate_act(g, act) * u);
   }
 }
 
 // bfloat16 rows whose length is a multiple of 8: eight elements (16 bytes) per thread.
 __global__ void silu_gate_bf16x8_kernel(uint4* __restrict__ out, const uint4* __restrict__ gu, int chunks,
-                                        size_t total) {
+                                        size_t total, int act) {
   size_t i = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   const size_t step = static_cast<size_t>(gridDim.x) * blockDim.x;
   for (; i < total; i += step) {
@@ -378,8 +381,8 @@ __global__ void silu_gate_bf16x8_kernel(uint4* __restrict__ out, const uint4* __
     for (int j = 0; j < 4; ++j) {
       const float g0 = __uint_as_float(gw[j] << 16), g1 = __uint_as_float(gw[j] & 0xffff0000u);
       const float u0 = __uint_as_float(uw[j] << 16), u1 = __uint_as_float(uw[j] & 0xffff0000u);
-      const float a0 = (g0 / (1.0f + expf(-g0))) * u0;
-      const float a1 = (g1 / (1.0f + expf(-g1))) * u1;
+      const float a0 = pylon_gate_act(g0, act) * u0;
+      const float a1 = pylon_gate_act(g1, act) * u1;
       r[j] = static_cast<uint32_t>(float_to_bf16_bits(a0)) | (static_cast<uint32_t>(float_to_bf16_bits(a1)) << 16);
     }
     out[i] = uint4{r[0], r[1], r[2], r[3]};
@@ -389,7 +392,8 @@ __global__ void silu_gate_bf16x8_kernel(uint4* __restrict__ out, const uint4* __
 // gate_up: [tokens, 2 * inter] of in_dtype; out: [tokens, inter] of out_dtype (float sums of a
 // product may come in as float and leave as bfloat16: one rounding, after the activation).
 extern "C" int pylon_silu_gate(void* out, int out_dtype, const void* gate_up, int in_dtype, int tokens, int inter,
-                               hipStream_t stream) {
+                               int act, hipStream_t stream) {
+  PYLON_REQUIRE(act == PYLON_ACT_SILU || act == PYLON_ACT_GELU, "silu_gate: unknown activation %d", act);
   PYLON_REQUIRE(pylon_valid_dtype(in_dtype) && pylon_valid_dtype(out_dtype), "silu_gate: unknown dtype");
   PYLON_REQUIRE(tokens >= 0 && inter > 0, "silu_gate: bad sizes tokens=%d inter=%d", tokens, inter);
   const size_t total = static_cast<size_t>(tokens) * inter;
@@ -400,14 +404,14 @@ extern "C" int pylon_silu_gate(void* out, int out_dtype, const void* gate_up, in
     size_t nblocks = (chunks_total + 255) / 256;
     if (nblocks > 65535u * 16u) nblocks = 65535u * 16u;
     hipLaunchKernelGGL(silu_gate_bf16x8_kernel, dim3((unsigned)nblocks), dim3(256), 0, stream, (uint4*)out,
-                       (const uint4*)gate_up, inter / 8, chunks_total);
+                       (const uint4*)gate_up, inter / 8, chunks_total, act);
     PYLON_LAUNCHED("silu_gate");
   }
   size_t blocks = (total + 255) / 256;
   if (blocks > 65535u * 16u) blocks = 65535u * 16u;
   dim3 grid((unsigned)blocks), block(256);
 #define GO(TI, TO) \
-  hipLaunchKernelGGL((silu_gate_kernel<TI, TO>), grid, block, 0, stream, (TO*)out, (const TI*)gate_up, inter, total)
+  hipLaunchKernelGGL((silu_gate_kernel<TI, TO>), grid, block, 0, stream, (TO*)out, (const TI*)gate_up, inter, total, act)
   if (in_dtype == PYLON_F32 && out_dtype == PYLON_F32) GO(float, float);
   else if (in_dtype == PYLON_F32) GO(float, bf16_t);
   else if (out_dtype == PYLON_F32) GO(bf16_t, float);

@@ -52,8 +52,6 @@ typedef float floatx4 __attribute__((ext_vector_type(4)));
 // chunks in flight would drain at every barrier.)
 __device__ __forceinline__ void gr_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
 
-__device__ __forceinline__ float gr_silu(float z) { return z / (1.0f + expf(-z)); }
-
 // vmcnt <= N (N < 64); the other counters are left alone.
 template <int N>
 __device__ __forceinline__ void gr_wait_loads() {
@@ -82,7 +80,7 @@ template <int MT, int CT, bool GLU, int WAVES, typename TO>
 __device__ __forceinline__ void gemm_rows_body(
     TO* __restrict__ out, const uint16_t* __restrict__ x, const uint16_t* __restrict__ w, int M, int N,
     int K, long long ldx, long long ldw, long long ldo, long long part_stride, int chunks_per_part,
-    int wg_cols, int group, int relu2) {
+    int wg_cols, int group, int variant) {
   typedef GrShape<MT, CT, WAVES> Shape;
   constexpr int QW = 4 / WAVES;  // quarters of every tile of x that a wave fills
   constexpr int STAGES = Shape::STAGES;
@@ -231,8 +229,8 @@ __device__ __forceinline__ void gemm_rows_body(
       floatx4 v = acc[j][t];
       if constexpr (GLU) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = gr_silu(acc[0][t][i]) * acc[1][t][i];
-      } else if (relu2) {
+        for (int i = 0; i < 4; ++i) v[i] = pylon_gate_act(acc[0][t][i], variant) * acc[1][t][i];
+      } else if (variant) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const float pos = fmaxf(v[i], 0.f);
@@ -262,7 +260,7 @@ template <int MT, int CT, bool GLU, int WAVES, typename TO>
 __global__ __launch_bounds__(WAVES* PYLON_WAVE) void gemm_rows_kernel(
     TO* __restrict__ out, const uint16_t* __restrict__ x, const uint16_t* __restrict__ w, int M, int N,
     int K, long long ldx, long long ldw, long long ldo, long long part_stride, int chunks_per_part,
-    int wg_cols, int groups, int row_split, int relu2) {
+    int wg_cols, int groups, int row_split, int variant) {
   // More than 64 rows of x go as two halves of `row_split` rows, each to workgroups of its
   // own that take the same columns: blockIdx.x counts eight groups of columns for the first
   // half, the same eight for the second, then the next eight, so that the two workgroups that
@@ -278,7 +276,7 @@ __global__ __launch_bounds__(WAVES* PYLON_WAVE) void gemm_rows_kernel(
     M = (M - half * row_split < row_split) ? M - half * row_split : row_split;
   }
   gemm_rows_body<MT, CT, GLU, WAVES, TO>(out, x, w, M, N, K, ldx, ldw, ldo, part_stride, chunks_per_part, wg_cols,
-                                         group, relu2);
+                                         group, variant);
 }
 
 // How a product is laid over the chip: wavefronts per workgroup, workgroups along the columns,
@@ -319,31 +317,31 @@ static GrLaunch gr_launch_shape(int M, int N, int parts, int col_tiles, int glu,
 template <int MT, int CT, bool GLU, int WAVES>
 static void launch_rows_waves(void* out, int out_dtype, const void* x, const void* w, int M, int N, int K,
                               long long ldx, long long ldw, long long ldo, int parts, long long part_stride,
-                              const GrLaunch& shape, int row_split, int relu2, hipStream_t stream) {
+                              const GrLaunch& shape, int row_split, int variant, hipStream_t stream) {
   const int chunks = (K + GR_CHUNK - 1) / GR_CHUNK;
   const int per_part = (chunks + parts - 1) / parts;
   dim3 grid(row_split > 0 ? 2 * ((shape.groups + 7) / 8 * 8) : shape.groups, parts), block(WAVES * PYLON_WAVE);
   if (out_dtype == PYLON_F32)
     hipLaunchKernelGGL((gemm_rows_kernel<MT, CT, GLU, WAVES, float>), grid, block, 0, stream, (float*)out,
                        (const uint16_t*)x, (const uint16_t*)w, M, N, K, ldx, ldw, ldo, part_stride, per_part,
-                       shape.wg_cols, shape.groups, row_split, relu2);
+                       shape.wg_cols, shape.groups, row_split, variant);
   else
     hipLaunchKernelGGL((gemm_rows_kernel<MT, CT, GLU, WAVES, bf16_t>), grid, block, 0, stream, (bf16_t*)out,
                        (const uint16_t*)x, (const uint16_t*)w, M, N, K, ldx, ldw, ldo, part_stride, per_part,
-                       shape.wg_cols, shape.groups, row_split, relu2);
+                       shape.wg_cols, shape.groups, row_split, variant);
 }
 
 // Workgroups of four waves, or of two where four would leave compute units without one.
 template <int MT, int CT, bool GLU>
 static void launch_rows(void* out, int out_dtype, const void* x, const void* w, int M, int N, int K,
                         long long ldx, long long ldw, long long ldo, int parts, long long part_stride,
-                        const GrLaunch& shape, int row_split, int relu2, hipStream_t stream) {
+                        const GrLaunch& shape, int row_split, int variant, hipStream_t stream) {
   if (shape.waves == 2)
     launch_rows_waves<MT, CT, GLU, 2>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, shape,
-                                      row_split, relu2, stream);
+                                      row_split, variant, stream);
   else
     launch_rows_waves<MT, CT, GLU, 4>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, shape,
-                                      row_split, relu2, stream);
+                                      row_split, variant, stream);
 }
 
 // What pylon_gemm_rows would launch for these arguments on a device of `units` compute units
@@ -367,7 +365,8 @@ extern "C" int pylon_gemm_rows_shape(int M, int N, int parts, int col_tiles, int
 // workgroups of its own); w: [N, ldw] bf16 (with glu: [2N, ldw], gate rows first, then
 // up rows); out: `parts` results [M, ldo] spaced part_stride elements apart (parts > 1 needs
 // float out and no glu).  col_tiles: tiles of 16 columns per wave, 1 or 2; with glu a wave
-// takes 16 gate rows and their 16 up rows; glu = 2: no gate, the result is max(x w^T, 0)^2.  waves: wavefronts per workgroup, 4 or 2 (0: two if
+// takes 16 gate rows and their 16 up rows, gated through silu (glu = 3: through gelu);
+// glu = 2: no gate, the result is max(x w^T, 0)^2.  waves: wavefronts per workgroup, 4 or 2 (0: two if
 // four would give fewer workgroups than half the device's compute units).  cols: columns per
 // workgroup, at most what its waves' tiles hold (0: the rule of gr_launch_shape); the sums do
 // not depend on it.
@@ -375,10 +374,11 @@ extern "C" int pylon_gemm_rows(void* out, int out_dtype, const void* x, const vo
                                long long ldx, long long ldw, long long ldo, int parts, long long part_stride,
                                int col_tiles, int glu, int waves, int cols, hipStream_t stream) {
   PYLON_REQUIRE(pylon_valid_dtype(out_dtype), "gemm_rows: unknown output dtype");
-  PYLON_REQUIRE(glu >= 0 && glu <= 2, "gemm_rows: unknown epilogue %d", glu);
-  const int relu2 = glu == 2 ? 1 : 0;
-  PYLON_REQUIRE(parts == 1 || !relu2, "gemm_rows: the squared relu needs the whole of K");
-  if (relu2) glu = 0;
+  PYLON_REQUIRE(glu >= 0 && glu <= 3, "gemm_rows: unknown epilogue %d", glu);
+  // 1: the squared relu of a product without a gate, or gelu instead of silu in one with
+  const int variant = glu >= 2 ? 1 : 0;
+  PYLON_REQUIRE(parts == 1 || glu != 2, "gemm_rows: the squared relu needs the whole of K");
+  glu &= 1;
   PYLON_REQUIRE(M >= 0 && M <= 128, "gemm_rows: takes at most 128 rows, got %d", M);
   PYLON_REQUIRE(N > 0 && K > 0, "gemm_rows: bad sizes N=%d K=%d", N, K);
   PYLON_REQUIRE(K % 8 == 0, "gemm_rows: K=%d must be a multiple of 8", K);
@@ -409,9 +409,9 @@ extern "C" int pylon_gemm_rows(void* out, int out_dtype, const void* x, const vo
                 "gemm_rows: %d columns per workgroup are more than the tiles of its %d waves hold", cols, shape.waves);
 #define GO(MT)                                                                                              \
   do {                                                                                                      \
-    if (glu) launch_rows<MT, 2, true>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, shape, row_split, relu2, stream); \
-    else if (col_tiles == 2) launch_rows<MT, 2, false>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, shape, row_split, relu2, stream); \
-    else launch_rows<MT, 1, false>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, shape, row_split, relu2, stream); \
+    if (glu) launch_rows<MT, 2, true>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, shape, row_split, variant, stream); \
+    else if (col_tiles == 2) launch_rows<MT, 2, false>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, shape, row_split, variant, stream); \
+    else launch_rows<MT, 1, false>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, shape, row_split, variant, stream); \
   } while (0)
   switch ((rows_each + 15) / 16) {
     case 1: GO(1); break;

@@ -38,7 +38,6 @@ __device__ __forceinline__ bf16x8 zero8() {
   return z;
 }
 
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
 
 // RT: 16-row tiles of w per workgroup (with GLU: RT tiles of gate rows and RT of up rows).
 // A wave multiplies every tile of w with every tile of x, so RT tiles of w pay for the rows of
@@ -46,7 +45,7 @@ __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z));
 template <int MT, int WAVES, bool GLU, int RT, typename TO>
 __global__ __launch_bounds__(WAVES* PYLON_WAVE) void gemm_skinny_kernel(
     TO* __restrict__ out, const uint16_t* __restrict__ x, const uint16_t* __restrict__ w, int M, int N,
-    int K, long long ldx, long long ldw, long long ldo, long long part_stride, int relu2) {
+    int K, long long ldx, long long ldw, long long ldo, long long part_stride, int variant) {
   constexpr int TILES = GLU ? 2 * RT : RT;  // row tiles of w per workgroup
   __shared__ floatx4 red[WAVES][TILES][MT][PYLON_WAVE];
   const int lane = threadIdx.x & (PYLON_WAVE - 1);
@@ -135,7 +134,7 @@ __global__ __launch_bounds__(WAVES* PYLON_WAVE) void gemm_skinny_kernel(
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             const int n = n0 + 16 * j + 4 * g + i;
-            if (n < N) dst[n] = from_float<TO>(silu_f(sum[j][i]) * sum[RT + j][i]);
+            if (n < N) dst[n] = from_float<TO>(pylon_gate_act(sum[j][i], variant) * sum[RT + j][i]);
           }
       } else {
 #pragma unroll
@@ -144,7 +143,7 @@ __global__ __launch_bounds__(WAVES* PYLON_WAVE) void gemm_skinny_kernel(
           for (int i = 0; i < 4; ++i) {
             const int n = n0 + 16 * j + 4 * g + i;
             const float pos = fmaxf(sum[j][i], 0.f);
-            if (n < N) dst[n] = from_float<TO>(relu2 ? pos * pos : sum[j][i]);
+            if (n < N) dst[n] = from_float<TO>(variant ? pos * pos : sum[j][i]);
           }
       }
     }
@@ -154,26 +153,26 @@ __global__ __launch_bounds__(WAVES* PYLON_WAVE) void gemm_skinny_kernel(
 template <int MT, int WAVES, bool GLU, int RT>
 static void launch_skinny(void* out, int out_dtype, const void* x, const void* w, int M, int N, int K,
                           long long ldx, long long ldw, long long ldo, int parts, long long part_stride,
-                          int relu2, hipStream_t stream) {
+                          int variant, hipStream_t stream) {
   constexpr int ROWS = 16 * RT;
   dim3 grid((N + ROWS - 1) / ROWS, parts), block(WAVES * PYLON_WAVE);
   if (out_dtype == PYLON_F32)
     hipLaunchKernelGGL((gemm_skinny_kernel<MT, WAVES, GLU, RT, float>), grid, block, 0, stream, (float*)out,
-                       (const uint16_t*)x, (const uint16_t*)w, M, N, K, ldx, ldw, ldo, part_stride, relu2);
+                       (const uint16_t*)x, (const uint16_t*)w, M, N, K, ldx, ldw, ldo, part_stride, variant);
   else
     hipLaunchKernelGGL((gemm_skinny_kernel<MT, WAVES, GLU, RT, bf16_t>), grid, block, 0, stream, (bf16_t*)out,
-                       (const uint16_t*)x, (const uint16_t*)w, M, N, K, ldx, ldw, ldo, part_stride, relu2);
+                       (const uint16_t*)x, (const uint16_t*)w, M, N, K, ldx, ldw, ldo, part_stride, variant);
 }
 
 template <int MT>
 static void launch_skinny_mt(void* out, int out_dtype, const void* x, const void* w, int M, int N, int K,
                              long long ldx, long long ldw, long long ldo, int parts,
-                             long long part_stride, int glu, int relu2, hipStream_t stream) {
+                             long long part_stride, int glu, int variant, hipStream_t stream) {
   // Four waves measured faster than eight at every shape of a 4B-class decoder; the
   // eight-wave form is kept for very long K only.
   const int steps = (K + SK_STEP - 1) / SK_STEP / parts;
   const bool wide = steps >= 512;
-#define GO(W, G, R) launch_skinny<MT, W, G, R>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, relu2, stream)
+#define GO(W, G, R) launch_skinny<MT, W, G, R>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, variant, stream)
   if (glu) {
     if (wide) GO(8, true, 1); else GO(4, true, 1);
   } else if (MT == 1 && parts == 1 && N >= 4096) {
@@ -188,15 +187,16 @@ static void launch_skinny_mt(void* out, int out_dtype, const void* x, const void
 
 // x: [M, ldx] bf16; w: [N, ldw] bf16 (with glu: [2N, ldw], gate rows first, then up rows);
 // out: `parts` results [M, ldo] spaced part_stride elements apart (parts > 1 needs float out
-// and no glu).  glu = 2: no gate, the result is max(x w^T, 0)^2.
+// and no glu).  glu = 3: gated through gelu instead of silu; glu = 2: no gate, the result is max(x w^T, 0)^2.
 extern "C" int pylon_gemm_skinny(void* out, int out_dtype, const void* x, const void* w, int M, int N,
                                  int K, long long ldx, long long ldw, long long ldo, int parts,
                                  long long part_stride, int glu, hipStream_t stream) {
   PYLON_REQUIRE(pylon_valid_dtype(out_dtype), "gemm_skinny: unknown output dtype");
-  PYLON_REQUIRE(glu >= 0 && glu <= 2, "gemm_skinny: unknown epilogue %d", glu);
-  const int relu2 = glu == 2 ? 1 : 0;
-  PYLON_REQUIRE(parts == 1 || !relu2, "gemm_skinny: the squared relu needs the whole of K");
-  if (relu2) glu = 0;
+  PYLON_REQUIRE(glu >= 0 && glu <= 3, "gemm_skinny: unknown epilogue %d", glu);
+  // 1: the squared relu of a product without a gate, or gelu instead of silu in one with
+  const int variant = glu >= 2 ? 1 : 0;
+  PYLON_REQUIRE(parts == 1 || glu != 2, "gemm_skinny: the squared relu needs the whole of K");
+  glu &= 1;
   PYLON_REQUIRE(M >= 0 && M <= 64, "gemm_skinny: takes at most 64 rows, got %d", M);
   PYLON_REQUIRE(N > 0 && K > 0, "gemm_skinny: bad sizes N=%d K=%d", N, K);
   PYLON_REQUIRE(K % 8 == 0, "gemm_skinny: K=%d must be a multiple of 8", K);
@@ -211,10 +211,10 @@ extern "C" int pylon_gemm_skinny(void* out, int out_dtype, const void* x, const 
                 "gemm_skinny: partial results overlap");
   if (M == 0) return 0;
   switch ((M + 15) / 16) {
-    case 1: launch_skinny_mt<1>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, glu, relu2, stream); break;
-    case 2: launch_skinny_mt<2>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, glu, relu2, stream); break;
-    case 3: launch_skinny_mt<3>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, glu, relu2, stream); break;
-    default: launch_skinny_mt<4>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, glu, relu2, stream); break;
+    case 1: launch_skinny_mt<1>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, glu, variant, stream); break;
+    case 2: launch_skinny_mt<2>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, glu, variant, stream); break;
+    case 3: launch_skinny_mt<3>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, glu, variant, stream); break;
+    default: launch_skinny_mt<4>(out, out_dtype, x, w, M, N, K, ldx, ldw, ldo, parts, part_stride, glu, variant, stream); break;
   }
   PYLON_LAUNCHED("gemm_skinny");
 }

@@ -11,8 +11,10 @@
 // expert_down: out[t] = sum_s weight[t, s] W_down[e_s] hidden[(t, s)] (+ gate[t] * shared[t]), float.
 // route_scored: the other way to choose: scores are the softmax over all router outputs; a
 //   correction is added to them for the choice only; the outputs form equal groups of neighbours of
-//   which only the best few (by their largest corrected score) may be chosen from; the weights are the
-//   chosen scores times a constant, not renormalised.  The last router outputs may be identity
+//   which only the best few (by their largest corrected score, or by the sum of their two largest) may be
+//   chosen from; the weights are the
+//   chosen scores times a constant, as they are or divided by their sum.  scoring 1: every output's own
+//   sigmoid instead of the softmax.  The last router outputs may be identity
 //   experts, whose output is the token's input itself: their weights are summed into one number per
 //   token, and the expert kernels pass over them.
 // Experts may also be plain, W_down act(W_up x) with act the square of relu (`act` 1).
@@ -109,9 +111,10 @@ extern "C" int pylon_route_top(int* experts, float* weights, float* shared_gate,
 __global__ void __launch_bounds__(256)
 route_scored_kernel(int* __restrict__ experts, float* __restrict__ weights, float* __restrict__ identity_weight,
                     const float* __restrict__ logits, long long row_stride, const float* __restrict__ correction,
-                    int tokens, int n_outputs, int n_experts, int top, int groups, int keep, float scale) {
+                    int tokens, int n_outputs, int n_experts, int top, int groups, int keep, float scale, int scoring,
+                    int group_two, int renormalize) {
   __shared__ float choice[4][MX_MAX_OUTPUTS];  // corrected scores, then -inf outside the kept groups
-  __shared__ float best_of[4][MX_MAX_OUTPUTS];  // every group's largest corrected score
+  __shared__ float best_of[4][MX_MAX_OUTPUTS];  // every group's score
   const int lane = threadIdx.x & (PYLON_WAVE - 1), wave = threadIdx.x / PYLON_WAVE;
   const int t = blockIdx.x * 4 + wave;
   if (t >= tokens) return;  // whole waves leave; only wave-level barriers follow
@@ -136,16 +139,20 @@ route_scored_kernel(int* __restrict__ experts, float* __restrict__ weights, floa
 #pragma unroll
   for (int i = 0; i < 8; ++i) {
     const int e = lane + PYLON_WAVE * i;
-    s[i] *= inv;
+    s[i] = scoring == 1 ? 1.0f / (1.0f + expf(-z[i])) : s[i] * inv;
     if (e < n_outputs) choice[wave][e] = s[i] + (correction != nullptr ? correction[e] : 0.f);
   }
   __builtin_amdgcn_wave_barrier();
   const int per_group = n_outputs / groups;
   if (keep < groups) {
     for (int g = lane; g < groups; g += PYLON_WAVE) {
-      float m = -INFINITY;
-      for (int k = 0; k < per_group; ++k) m = fmaxf(m, choice[wave][g * per_group + k]);
-      best_of[wave][g] = m;
+      float m = -INFINITY, second = -INFINITY;
+      for (int k = 0; k < per_group; ++k) {
+        const float v = choice[wave][g * per_group + k];
+        second = fmaxf(second, fminf(v, m));
+        m = fmaxf(m, v);
+      }
+      best_of[wave][g] = group_two && per_group > 1 ? m + second : m;
     }
     __builtin_amdgcn_wave_barrier();
     // a group is kept if fewer than `keep` groups come before it (a larger score, or an equal one
@@ -168,6 +175,7 @@ route_scored_kernel(int* __restrict__ experts, float* __restrict__ weights, floa
     const int e = lane + PYLON_WAVE * i;
     c[i] = e < n_outputs ? choice[wave][e] : -INFINITY;
   }
+  float sum_chosen = 0.f;
   float ident = 0.f;  // lane 0 adds up the identity experts' weights, in the order of the choices
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY, best_s = 0.f;
@@ -202,7 +210,13 @@ route_scored_kernel(int* __restrict__ experts, float* __restrict__ weights, floa
       experts[static_cast<size_t>(t) * top + k] = none ? n_outputs : best_e;
       weights[static_cast<size_t>(t) * top + k] = identity ? 0.f : w;
       if (identity) ident += w;
+      sum_chosen += none ? 0.f : best_s;
     }
+  }
+  if (lane == 0 && renormalize) {  // lane 0 wrote the weights itself
+    const float by = 1.0f / (sum_chosen + 1e-20f);
+    for (int k = 0; k < top; ++k) weights[static_cast<size_t>(t) * top + k] *= by;
+    ident *= by;
   }
   if (lane == 0 && identity_weight != nullptr) identity_weight[t] = ident;
 }
@@ -210,10 +224,14 @@ route_scored_kernel(int* __restrict__ experts, float* __restrict__ weights, floa
 // logits: float [tokens, n_outputs], rows row_stride apart; correction: null or float [n_outputs];
 // the first n_experts outputs are experts, the others identities.  experts int [tokens, top] (an
 // identity keeps its index, >= n_experts), weights float [tokens, top] (nothing for an identity),
-// identity_weight float [tokens] (null only if n_outputs == n_experts).
+// identity_weight float [tokens] (null only if n_outputs == n_experts).  scoring 0: softmax over all outputs,
+// 1: every output's sigmoid; group_two: a group's score is the sum of its two largest corrected scores, not
+// its largest; renormalize: the weights are divided by their sum (+ 1e-20) before the scale.
 extern "C" int pylon_route_scored(int* experts, float* weights, float* identity_weight, const float* logits,
                                   long long row_stride, const float* correction, int tokens, int n_outputs,
-                                  int n_experts, int top, int groups, int keep, float scale, hipStream_t stream) {
+                                  int n_experts, int top, int groups, int keep, float scale, int scoring, int group_two,
+                                  int renormalize, hipStream_t stream) {
+  PYLON_REQUIRE(scoring == 0 || scoring == 1, "route_scored: unknown scoring %d", scoring);
   PYLON_REQUIRE(tokens >= 0 && n_outputs >= 1 && n_outputs <= MX_MAX_OUTPUTS,
                 "route_scored: 1 to %d router outputs, got %d", MX_MAX_OUTPUTS, n_outputs);
   PYLON_REQUIRE(n_experts >= 0 && n_experts <= n_outputs, "route_scored: %d experts among %d outputs", n_experts, n_outputs);
@@ -226,7 +244,7 @@ extern "C" int pylon_route_scored(int* experts, float* weights, float* identity_
   if (tokens == 0) return 0;
   hipLaunchKernelGGL(route_scored_kernel, dim3((tokens + 3) / 4), dim3(256), 0, stream, experts, weights,
                      identity_weight, logits, row_stride, correction, tokens, n_outputs, n_experts, top, groups, keep,
-                     scale);
+                     scale, scoring, group_two, renormalize);
   PYLON_LAUNCHED("route_scored");
 }
 

@@ -4,7 +4,7 @@
 //   d = sum_p delta[p]                      (the sublayer's output, maybe as partial sums)
 //   x = resid + post_gain * d / rms(d)      (rms(v) = sqrt(mean(v^2) + eps); without post_gain: x = resid + d)
 //   or, with a bias and a scale per element (a projection's bias that was left for here, a layer's
-//   learned scale of its sublayers' outputs): x = resid + scale * (d + bias)
+//   learned scale of its sublayers' outputs): x = resid + factor * scale * (d + bias), factor one number of the launch
 //   out = gain * x / rms(x)                 (gain: one number, or one per element)
 //
 // All of it in float; `out` is rounded once on the store.  One workgroup per output row, the
@@ -20,7 +20,8 @@ __global__ void add_normed_rmsnorm_kernel(TO* __restrict__ out, float* resid, co
                                           int n_delta, long long delta_stride, const float* __restrict__ post_gain,
                                           float post_eps, const float* __restrict__ gain, int gain_stride,
                                           const int* __restrict__ row_idx, int dim, float eps, int write_resid,
-                                          const float* __restrict__ delta_scale, const float* __restrict__ delta_bias) {
+                                          const float* __restrict__ delta_scale, const float* __restrict__ delta_bias,
+                                          float factor) {
   __shared__ float scratch[16];
   const int r_out = blockIdx.x;
   const int r_in = row_idx ? row_idx[r_out] : r_out;
@@ -82,7 +83,8 @@ __global__ void add_normed_rmsnorm_kernel(TO* __restrict__ out, float* resid, co
       const int i = threadIdx.x + n * blockDim.x;
       x[n] = 0.f;
       if (i < dim) {
-        x[n] = delta_scale ? fmaf(delta_scale[i], d[n], xr[i]) : xr[i] + (d[n] * mult) * pg;
+        x[n] = delta_scale ? fmaf(factor * delta_scale[i], d[n], xr[i])
+                           : (post_gain ? xr[i] + (d[n] * mult) * pg : fmaf(factor, d[n], xr[i]));
         if (write_resid) xr[i] = x[n];
       }
     }
@@ -114,8 +116,9 @@ __global__ void add_normed_rmsnorm_kernel(TO* __restrict__ out, float* resid, co
 extern "C" int pylon_add_normed_rmsnorm(void* out, int out_dtype, float* resid, const void* delta, int delta_dtype,
                                         int n_delta, long long delta_stride, const float* post_gain, float post_eps,
                                         const float* gain, int gain_stride, const int* row_idx, int rows, int dim,
-                                        float eps, const float* delta_scale, const float* delta_bias,
+                                        float eps, const float* delta_scale, const float* delta_bias, float factor,
                                         hipStream_t stream) {
+  PYLON_REQUIRE(factor == 1.0f || post_gain == nullptr, "add_normed_rmsnorm: a normed output has no further factor");
   PYLON_REQUIRE(pylon_valid_dtype(out_dtype) && pylon_valid_dtype(delta_dtype), "add_normed_rmsnorm: unknown dtype");
   PYLON_REQUIRE(rows >= 0 && dim > 0 && dim <= 16384, "add_normed_rmsnorm: rows of 1 to 16384 elements, got %d", dim);
   PYLON_REQUIRE(n_delta >= 1 && (gain_stride == 0 || gain_stride == 1), "add_normed_rmsnorm: bad delta count or gain stride");
@@ -133,7 +136,7 @@ extern "C" int pylon_add_normed_rmsnorm(void* out, int out_dtype, float* resid, 
 #define GO(TD, TO, PER, ND)                                                                                     \
   hipLaunchKernelGGL((add_normed_rmsnorm_kernel<TD, TO, PER, ND>), grid, block, 0, stream, (TO*)out, resid,     \
                      (const TD*)delta, n_delta, delta_stride, post_gain, post_eps, gain, gain_stride, row_idx,  \
-                     dim, eps, write_resid, delta_scale, delta_bias)
+                     dim, eps, write_resid, delta_scale, delta_bias, factor)
 #define PICK(TD, TO, ND)              \
   do {                                \
     if (per <= 4) GO(TD, TO, 4, ND);      \

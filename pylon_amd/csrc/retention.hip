@@ -14,8 +14,11 @@
 // so a request's results do not depend on how it was cut into steps or what shared a step.
 #include "common.h"
 
-template <typename T, int NI, int THREADS>
-__global__ __launch_bounds__(THREADS) void retention_recurrent_kernel(T* __restrict__ out, const T* __restrict__ proj, long long ld,
+//
+// FORM 1 (lightning attention): q, k and v pass through silu (rounded to the model's type) instead of being
+// rotated and scaled, and o_t leaves as floats, unnormed and ungated.
+template <typename T, int NI, int THREADS, int FORM>
+__global__ __launch_bounds__(THREADS) void retention_recurrent_kernel(void* __restrict__ out_any, const T* __restrict__ proj, long long ld,
                                            int q_off, int k_off, int v_off, int g_off, float* state,
                                            const float* __restrict__ decay, const float* __restrict__ inv_freq,
                                            int rot_dims, const int* __restrict__ positions,
@@ -42,13 +45,15 @@ __global__ __launch_bounds__(THREADS) void retention_recurrent_kernel(T* __restr
   const int half = rot_dims / 2;
   for (int t = begin; t < end; ++t) {
     const T* pr = proj + static_cast<size_t>(t) * ld;
-    const float pos = static_cast<float>(positions[t]);
+    const float pos = FORM == 0 ? static_cast<float>(positions[t]) : 0.f;
     for (int e = tid; e < 2 * dim; e += blockDim.x) {
       const bool is_k = e >= dim;
       const int d = is_k ? e - dim : e;
       const T* src = pr + (is_k ? k_off : q_off) + head * dim;
       float v = to_float(src[d]);
-      if (d < rot_dims) {
+      if (FORM == 1) {
+        v = to_float(from_float<T>(pylon_silu(v)));
+      } else if (d < rot_dims) {
         const int pair = d < half ? d : d - half;
         const float angle = pos * inv_freq[pair];
         float sn, cs;
@@ -60,7 +65,8 @@ __global__ __launch_bounds__(THREADS) void retention_recurrent_kernel(T* __restr
       else qs[d] = v;
     }
     __syncthreads();
-    const float vj = to_float(pr[v_off + head * vdim + j]);
+    float vj = to_float(pr[v_off + head * vdim + j]);
+    if (FORM == 1) vj = to_float(from_float<T>(pylon_silu(vj)));
     float acc = 0.f;
     if (owner) {
 #pragma unroll
@@ -79,6 +85,12 @@ __global__ __launch_bounds__(THREADS) void retention_recurrent_kernel(T* __restr
       for (int p = 0; p < ip_count; ++p) o += part[p * vdim + j];
       sq = o * o;
     }
+    if (FORM == 1) {
+      // (the next token's q and k are written behind the barrier above, its parts behind the next one)
+      if (ip == 0) static_cast<float*>(out_any)[(static_cast<size_t>(t) * heads + head) * vdim + j] = o;
+      continue;
+    }
+    T* out = static_cast<T*>(out_any);
     const float total = block_sum(sq, red);  // two barriers inside: qs, ks and part are free again after it
     if (ip == 0) {
       const float inv = 1.0f / sqrtf(total / static_cast<float>(vdim) + eps);
@@ -95,14 +107,16 @@ __global__ __launch_bounds__(THREADS) void retention_recurrent_kernel(T* __restr
 
 // proj: [tokens, ld] of dtype, one row per token holding q (heads * dim elements from q_off),
 // k (from k_off), v (heads * vdim from v_off) and the gate g (heads * vdim from g_off).
-// out: [tokens, heads * vdim] of dtype.  state: float [slots, heads, dim, vdim].
+// out: [tokens, heads * vdim] of dtype (form 1: of float; no gate, no rotation, k_scale 1).  state: float [slots, heads, dim, vdim].
 // decay: float [heads]; inv_freq: float [rot_dims / 2] (null when rot_dims is 0).
 // The host guarantees row_slots < slots, one position per token and row_start[rows] <= tokens.
 extern "C" int pylon_retention_recurrent(void* out, const void* proj, int dtype, long long ld, int q_off, int k_off,
                                          int v_off, int g_off, float* state, const float* decay,
                                          const float* inv_freq, int rot_dims, const int* positions,
                                          const int* row_start, const int* row_slots, int rows, int heads, int dim,
-                                         int vdim, float eps, float k_scale, hipStream_t stream) {
+                                         int vdim, float eps, float k_scale, int form, hipStream_t stream) {
+  PYLON_REQUIRE(form == 0 || (form == 1 && rot_dims == 0 && k_scale == 1.0f),
+                "retention: form %d, or a rotation or a scale of k in the form that has none", form);
   PYLON_REQUIRE(pylon_valid_dtype(dtype), "retention: unknown dtype");
   PYLON_REQUIRE(rows >= 0 && heads > 0 && dim > 0 && vdim > 0, "retention: bad sizes");
   PYLON_REQUIRE(vdim <= 256 && dim <= 1024, "retention: heads of up to 1024 key and 256 value elements, got %d and %d",
@@ -121,15 +135,20 @@ extern "C" int pylon_retention_recurrent(void* out, const void* proj, int dtype,
   PYLON_REQUIRE(per <= 64, "retention: a head of %d x %d does not fit a workgroup's registers", dim, vdim);
   dim3 grid(rows, heads), block((vdim * ip_count + PYLON_WAVE - 1) / PYLON_WAVE * PYLON_WAVE);
   const size_t lds = sizeof(float) * (2 * dim + ip_count * vdim + 16);
-#define GO(T, NI)                                                                                              \
+#define GO2(T, NI, FORM)                                                                                            \
   if (block.x <= 256)                                                                                          \
-    hipLaunchKernelGGL((retention_recurrent_kernel<T, NI, 256>), grid, block, lds, stream, (T*)out, (const T*)proj, ld, \
+    hipLaunchKernelGGL((retention_recurrent_kernel<T, NI, 256, FORM>), grid, block, lds, stream, out, (const T*)proj, ld, \
                        q_off, k_off, v_off, g_off, state, decay, inv_freq, rot_dims, positions, row_start,      \
                        row_slots, heads, dim, vdim, ip_count, eps, k_scale);                                    \
   else                                                                                                         \
-    hipLaunchKernelGGL((retention_recurrent_kernel<T, NI, 1024>), grid, block, lds, stream, (T*)out, (const T*)proj, ld, \
+    hipLaunchKernelGGL((retention_recurrent_kernel<T, NI, 1024, FORM>), grid, block, lds, stream, out, (const T*)proj, ld, \
                      q_off, k_off, v_off, g_off, state, decay, inv_freq, rot_dims, positions, row_start,        \
                      row_slots, heads, dim, vdim, ip_count, eps, k_scale)
+#define GO(T, NI)                     \
+  do {                                \
+    if (form == 0) { GO2(T, NI, 0); } \
+    else { GO2(T, NI, 1); }           \
+  } while (0)
 #define PICK(T)                 \
   do {                          \
     if (per <= 4) GO(T, 4);     \
@@ -140,5 +159,6 @@ extern "C" int pylon_retention_recurrent(void* out, const void* proj, int dtype,
   else PICK(bf16_t);
 #undef PICK
 #undef GO
+#undef GO2
   PYLON_LAUNCHED("retention_recurrent");
 }

@@ -10,6 +10,7 @@ tokens), "logits" parts after the head (``forward(logits, ctx) -> logits``, floa
 per wanted token; under graph replay they must write in place).  A schedule entry with
 ``add_embedding`` has the embedded tokens (after the stream parts) added to the stream once more
 before its run: how a model that runs a stretch of layers several times feeds every further pass.
+Before an entry with ``begins_pass`` the model's "pass" part changes the stream instead.
 A model may keep the residual stream in several copies (``ModelSpec.streams``), ``[copies, tokens,
 dim]``: they start as the embedded tokens, the layers' arrangement says how they change, and the final
 norm reads their sum.
@@ -43,6 +44,12 @@ class Model(Part):
                              f"{sorted({layer.streams for layer in spec.layers})}")
         if spec.streams > 1 and (spec.stream_parts or any(self.embedding_again)):
             raise ValueError("parts on the embedded tokens and tokens added again need a residual stream in one copy")
+        begins = [(i, e.begins_pass) for i, e in enumerate(spec.schedule) if e.begins_pass is not None]
+        if begins and (spec.pass_entry is None or spec.streams > 1):
+            raise ValueError("runs that begin a pass need the model's pass_entry and a residual stream in one copy")
+        if any(not 0 <= t < spec.pass_entry.times for _, t in begins):
+            raise ValueError(f"a pass is numbered 0 to {spec.pass_entry.times - 1}")
+        self.begins_pass = dict(begins)
         self.add_param("embed", (spec.vocab_size, spec.hidden_size), dtype, device)
         if not spec.tie_word_embeddings:
             self.add_param("lm_head", (spec.vocab_size, spec.hidden_size), dtype, device)
@@ -51,6 +58,9 @@ class Model(Part):
             block = build_part("block", layer, dtype=dtype, device=device)
             self.blocks.append(block)
             self.add_child(f"layers.{index}", block)
+        self.pass_entry = None
+        if spec.pass_entry is not None:
+            self.pass_entry = self.add_child("pass_entry", build_part("pass", spec.pass_entry, dtype=dtype, device=device))
         self.final_norm = self.add_child(
             "final_norm", build_part("norm", spec.final_norm, dtype=dtype, device=device)
         )
@@ -109,11 +119,13 @@ class Model(Part):
         for part in self.stream_parts:
             resid = part.forward(resid, ctx)
         # a schedule may add the embedded tokens to the stream again before some of its runs
-        embedded = resid.clone() if any(self.embedding_again) else None
+        embedded = resid.clone() if any(self.embedding_again) or self.begins_pass else None
         delta = None
         for run, ((layer, cache_id, stores), again) in enumerate(zip(self.schedule, self.embedding_again)):
             if again:
                 ops.residual_add(resid, embedded)  # the pending output of the run before follows in the norm
+            if run in self.begins_pass:
+                resid, delta = self.pass_entry.forward(resid, delta, embedded, self.begins_pass[run], ctx)
             cache = ctx.cache(cache_id)
             if not stores:
                 # the lender's keys and values, the run's own fixed-size state

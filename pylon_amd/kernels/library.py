@@ -27,13 +27,16 @@ P, I, F, L = c_void_p, c_int, c_float, c_longlong
 _SIGNATURES = {
     "pylon_embed": [P, P, I, P, P, I, I, I, F, I, P],
     "pylon_rmsnorm": [P, I, P, I, P, P, I, I, F, P],
-    "pylon_add_rmsnorm": [P, I, P, P, I, I, L, P, P, I, I, F, P],
+    "pylon_add_rmsnorm": [P, I, P, P, I, I, L, P, P, I, I, F, F, P],
     "pylon_residual_add": [P, P, I, L, P],
-    "pylon_silu_gate": [P, I, P, I, I, I, P],
+    "pylon_silu_gate": [P, I, P, I, I, I, I, P],
     "pylon_qkv_prepare": [P, P, P, P, I, L, P, P, F, P, I, P, P, I, I, I, I, I, P],
     "pylon_paged_attention": [P, P, P, P, I, P, I, P, P, I, I, I, I, I, I, F, I, L, P, P, I, I, I, F, P, I, P],
     "pylon_attention_sink": [P, P, L, P, P, P, I, P, P, I, I, I, I, I, I, F, P, I, I, I, P, L, I, I, F, P, P],
-    "pylon_add_normed_rmsnorm": [P, I, P, P, I, I, L, P, F, P, I, P, I, I, F, P, P, P],
+    "pylon_add_normed_rmsnorm": [P, I, P, P, I, I, L, P, F, P, I, P, I, I, F, P, P, F, P],
+    "pylon_norm_gate": [P, I, P, P, P, L, I, I, F, I, P],
+    "pylon_pass_join": [P, I, P, P, I, I, L, F, P, I, I, P],
+    "pylon_pass_begin": [P, P, I, L, P, I, I, P],
     "pylon_depth_mix": [P, I, P, P, I, I, L, P, P, P, L, I, P, P, I, I, F, P],
     "pylon_stream_norm": [P, I, P, L, I, P, I, I, L, P, P, P, P, P, I, I, F, I, P],
     "pylon_relu2": [P, I, P, I, L, P],
@@ -41,8 +44,8 @@ _SIGNATURES = {
     "pylon_gla_chunked": [P, P, L, I, I, I, I, I, I, P, P, F, P, P, P, P, P, I, I, I, I, F, F, I, P, L, P, L, P],
     "pylon_short_conv": [P, I, P, I, P, I, P, P, P, I, I, I, I, L, I, P],
     "pylon_token_shift": [P, I, P, I, P, P, P, P, I, I, I, P],
-    "pylon_retention_recurrent": [P, P, I, L, I, I, I, I, P, P, P, I, P, P, P, I, I, I, I, F, F, P],
-    "pylon_retention_chunked": [P, P, L, I, I, I, I, P, P, P, I, P, P, P, I, I, I, I, F, F, I, P, L, P],
+    "pylon_retention_recurrent": [P, P, I, L, I, I, I, I, P, P, P, I, P, P, P, I, I, I, I, F, F, I, P],
+    "pylon_retention_chunked": [P, P, L, I, I, I, I, P, P, P, I, P, P, P, I, I, I, I, F, F, I, P, L, I, I, P],
     "pylon_kv_store": [P, P, P, I, L, I, I, P, I, I, I, I, P],
     "pylon_qkv_bias_store": [P, P, P, I, P, I, L, P, P, I, I, I, I, I, I, P],
     "pylon_gated_act": [P, I, P, I, I, I, F, F, F, P, P],
@@ -70,7 +73,7 @@ _SIGNATURES = {
     "pylon_head_project": [P, L, I, P, I, L, I, P, I, P, P, L, I, I, I, I, I, P],
     "pylon_gate_heads": [P, I, P, L, I, P],
     "pylon_route_top": [P, P, P, P, L, P, I, I, I, I, P],
-    "pylon_route_scored": [P, P, P, P, L, P, I, I, I, I, I, I, F, P],
+    "pylon_route_scored": [P, P, P, P, L, P, I, I, I, I, I, I, F, I, I, I, P],
     "pylon_expert_gate_up": [P, P, I, L, P, I, L, P, I, I, I, I, I, I, P, P],
     "pylon_expert_down": [P, P, I, P, I, L, P, P, P, P, I, I, I, I, I, P, L, P, P],
     "pylon_softcap": [P, L, F, P],

@@ -97,8 +97,8 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, *, out_dtype=None
 
 def add_rmsnorm(resid: torch.Tensor, delta: Optional[torch.Tensor], weight: torch.Tensor, eps: float,
                 out_dtype: torch.dtype, *, row_idx: Optional[torch.Tensor] = None,
-                out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``resid += delta`` (float32, in place) and the RMSNorm of the sum.
+                out: Optional[torch.Tensor] = None, factor: float = 1.0) -> torch.Tensor:
+    """``resid += factor * delta`` (float32, in place) and the RMSNorm of the sum.
 
     ``delta`` has the residual's shape, or is a stack ``[parts, tokens, dim]`` of partial
     sums that are added up first.  With ``row_idx`` only those rows are normed and
@@ -126,7 +126,7 @@ def add_rmsnorm(resid: torch.Tensor, delta: Optional[torch.Tensor], weight: torc
               _dev(resid, "resid", torch.float32), _dev(delta, "delta"),
               dtype_code(delta.dtype) if delta is not None else F32, n_delta, delta_stride,
               _dev(weight, "weight", torch.float32), _dev(row_idx, "row_idx", torch.int32),
-              rows, dim, float(eps), _stream())
+              rows, dim, float(eps), float(factor), _stream())
     return out
 
 
@@ -138,10 +138,14 @@ def residual_add(resid: torch.Tensor, delta: torch.Tensor) -> torch.Tensor:
     return resid
 
 
+GATE_ACTS = {"silu": 0, "gelu_tanh": 1}  # activations of a gated feed-forward's gate
+
+
 def silu_gate(gate_up: torch.Tensor, *, out_dtype: Optional[torch.dtype] = None,
-              out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``silu(gate_up[:, :I]) * gate_up[:, I:]`` for a ``[tokens, 2I]`` input; the result may
-    have another element type than the input (float32 sums in, bfloat16 out: one rounding)."""
+              out: Optional[torch.Tensor] = None, act: str = "silu") -> torch.Tensor:
+    """``act(gate_up[:, :I]) * gate_up[:, I:]`` for a ``[tokens, 2I]`` input (``act``: silu, or the
+    tanh form of gelu); the result may have another element type than the input (float32 sums in,
+    bfloat16 out: one rounding)."""
     if gate_up.dim() != 2 or gate_up.shape[1] % 2:
         raise KernelError("silu_gate takes a [tokens, 2*I] input")
     tokens, two_i = gate_up.shape
@@ -152,7 +156,7 @@ def silu_gate(gate_up: torch.Tensor, *, out_dtype: Optional[torch.dtype] = None,
     elif out.shape != (tokens, inter) or out.dtype != out_dtype:
         raise KernelError("silu_gate: out has the wrong shape or dtype")
     _lib.call("pylon_silu_gate", _dev(out, "out"), dtype_code(out.dtype), _dev(gate_up, "gate_up"),
-              dtype_code(gate_up.dtype), tokens, inter, _stream())
+              dtype_code(gate_up.dtype), tokens, inter, GATE_ACTS[act], _stream())
     return out
 
 
@@ -379,7 +383,7 @@ def add_normed_rmsnorm(resid: torch.Tensor, delta: Optional[torch.Tensor], gain:
                        out_dtype: Optional[torch.dtype], *, post_gain: Optional[torch.Tensor] = None,
                        post_eps: float = 0.0, row_idx: Optional[torch.Tensor] = None,
                        delta_scale: Optional[torch.Tensor] = None,
-                       delta_bias: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+                       delta_bias: Optional[torch.Tensor] = None, factor: float = 1.0) -> Optional[torch.Tensor]:
     """``resid += post_gain * d / rms(d)`` (``d`` = ``delta``, or the sum of a stack of float32
     partial sums; without ``post_gain``: ``resid += d``), in float32 and in place, then
     ``gain * resid / rms(resid)`` in ``out_dtype``, with ``rms(v) = sqrt(mean(v^2) + eps)``.
@@ -387,7 +391,7 @@ def add_normed_rmsnorm(resid: torch.Tensor, delta: Optional[torch.Tensor], gain:
     With ``row_idx`` only those rows are normed and ``resid`` is left as it is; with
     ``gain`` None only the sum is formed.  ``delta_bias`` (float32 ``[dim]``) is added to ``d``
     first; with ``delta_scale`` (float32 ``[dim]``, not together with ``post_gain``) the sum is
-    ``resid += delta_scale * d``."""
+    ``resid += delta_scale * d``.  ``factor`` multiplies what is added (not together with ``post_gain``)."""
     if resid.dim() != 2:
         raise KernelError("add_normed_rmsnorm takes a 2-D residual")
     dim = resid.shape[1]
@@ -419,8 +423,61 @@ def add_normed_rmsnorm(resid: torch.Tensor, delta: Optional[torch.Tensor], gain:
               dtype_code(delta.dtype) if delta is not None else F32, n_delta, delta_stride,
               _dev(post_gain, "post_gain", torch.float32), float(post_eps), _dev(gain, "gain", torch.float32),
               gain_stride, _dev(row_idx, "row_idx", torch.int32), rows, dim, float(eps),
-              _dev(delta_scale, "delta_scale", torch.float32), _dev(delta_bias, "delta_bias", torch.float32), _stream())
+              _dev(delta_scale, "delta_scale", torch.float32), _dev(delta_bias, "delta_bias", torch.float32), float(factor),
+              _stream())
     return out
+
+
+def norm_gate(x: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, eps: float, *, act: str = "sigmoid") -> torch.Tensor:
+    """``x / sqrt(mean(x^2) + eps) * weight * act(gate)`` row by row: float32 ``x`` ``[tokens, dim]`` (the
+    heads of a mixer side by side), ``gate`` ``[tokens, dim]`` (maybe a slice of a fused projection's rows)
+    of the type the result gets.  ``act``: sigmoid or silu."""
+    if x.dim() != 2 or gate.shape != x.shape or gate.stride(1) != 1:
+        raise KernelError("norm_gate takes [tokens, dim] rows and gates of the same shape")
+    rows, dim = x.shape
+    if weight.shape != (dim,):
+        raise KernelError(f"norm_gate: weight has shape {tuple(weight.shape)}, expected ({dim},)")
+    if not gate.is_cuda:
+        raise KernelError("gate must live on the GPU; there is no CPU path")
+    out = torch.empty((rows, dim), dtype=gate.dtype, device=x.device)
+    _lib.call("pylon_norm_gate", _dev(out, "out"), dtype_code(out.dtype), _dev(x, "x", torch.float32),
+              _dev(weight, "weight", torch.float32), gate.data_ptr(), gate.stride(0), rows, dim, float(eps),
+              {"sigmoid": 0, "silu": 1}[act], _stream())
+    return out
+
+
+def pass_join(resid: torch.Tensor, delta: Optional[torch.Tensor], embedded: torch.Tensor, out_dtype: torch.dtype, *,
+              factor: float = 1.0) -> torch.Tensor:
+    """``[tokens, 2 dim]`` rows ``[x | embedded]`` in ``out_dtype`` with ``x = resid + factor * delta``
+    (``delta`` None, ``[tokens, dim]``, or a stack of float32 partial sums); ``resid`` is left as it is."""
+    if resid.dim() != 2 or embedded.shape != resid.shape:
+        raise KernelError("pass_join takes a 2-D residual and embedded tokens of its shape")
+    n_delta, delta_stride = 1, 0
+    if delta is not None:
+        if delta.shape[-2:] != resid.shape or delta.dim() not in (2, 3):
+            raise KernelError("pass_join: delta and resid differ in shape")
+        if delta.dim() == 3:
+            n_delta, delta_stride = delta.shape[0], delta.shape[1] * delta.shape[2]
+    rows, dim = resid.shape
+    out = torch.empty((rows, 2 * dim), dtype=out_dtype, device=resid.device)
+    _lib.call("pylon_pass_join", _dev(out, "out"), dtype_code(out.dtype), _dev(resid, "resid", torch.float32),
+              _dev(delta, "delta"), F32 if delta is None else dtype_code(delta.dtype), n_delta, delta_stride,
+              float(factor), _dev(embedded, "embedded", torch.float32), rows, dim, _stream())
+    return out
+
+
+def pass_begin(resid: torch.Tensor, product: torch.Tensor, step: Optional[torch.Tensor]) -> torch.Tensor:
+    """``resid = product + step`` (float32, in place; ``product`` ``[tokens, dim]`` or a stack of partial
+    sums; ``step`` None or ``[dim]``)."""
+    if product.dtype != torch.float32 or product.shape[-2:] != resid.shape or product.dim() not in (2, 3):
+        raise KernelError("pass_begin takes a float32 product of the residual's shape, or partial sums of one")
+    rows, dim = resid.shape
+    if step is not None and step.shape != (dim,):
+        raise KernelError("pass_begin: step is one number per element")
+    parts = product.shape[0] if product.dim() == 3 else 1
+    _lib.call("pylon_pass_begin", _dev(resid, "resid", torch.float32), _dev(product, "product"), parts, rows * dim,
+              _dev(step, "step", torch.float32), rows, dim, _stream())
+    return resid
 
 
 def depth_mix(resid: torch.Tensor, delta: Optional[torch.Tensor], streams: torch.Tensor, index: int,
@@ -573,18 +630,29 @@ def short_conv(h: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tens
 
 
 RETENTION_CHUNK = 32
+RETENTION_FORMS = {"retention": 0, "lightning": 1}
 RETENTION_PARALLEL_BYTES = 1 << 29  # the most memory the chunks' states may take
 
 
 def retention_chunk_parallel(rows: int, heads: int, dim: int, vdim: int, max_count: int,
                              units: Optional[int] = None) -> bool:
-    """Whether chunked retention takes one workgroup a chunk: when one workgroup a (row, head) would
-    leave most compute units idle, the rows are long enough for the two extra launches to pay, and
-    the chunks' states (float32, ``dim x vdim`` a chunk and head) fit a bound."""
+    """Whether chunked retention takes one workgroup a stretch of chunks: when one workgroup a (row, head)
+    would leave most compute units idle, the rows are long enough for the two extra launches to pay, and
+    the stretches' states (float32, ``dim x vdim`` a stretch and head) fit a bound."""
     units = units or _lib.compute_units()
     chunks = -(-max_count // RETENTION_CHUNK)
+    stretches = -(-chunks // retention_chunk_span(rows, heads, max_count, units))
     return (rows * heads * 2 <= units and chunks >= 4
-            and rows * heads * chunks * dim * vdim * 4 <= RETENTION_PARALLEL_BYTES)
+            and rows * heads * stretches * dim * vdim * 4 <= RETENTION_PARALLEL_BYTES)
+
+
+def retention_chunk_span(rows: int, heads: int, max_count: int, units: Optional[int] = None) -> int:
+    """Chunks of 32 tokens a workgroup of the chunk-parallel form walks: as many as still leave two
+    workgroups for every compute unit (a stretch's state is written, scanned and read once, so longer
+    stretches move fewer bytes)."""
+    units = units or _lib.compute_units()
+    chunks = -(-max_count // RETENTION_CHUNK)
+    return max(1, rows * heads * chunks // (2 * units))
 
 
 def retention_chunked_ok(dtype: torch.dtype, *, dim: int, vdim: int, rot_dims: int) -> bool:
@@ -597,14 +665,21 @@ def retention_recurrent(proj: torch.Tensor, state: torch.Tensor, decay: torch.Te
                         inv_freq: Optional[torch.Tensor], positions: torch.Tensor, row_start: torch.Tensor,
                         row_slots: torch.Tensor, *, rows: int, heads: int, dim: int, vdim: int, rot_dims: int,
                         eps: float, k_scale: float, chunked: bool = False,
-                        max_count: Optional[int] = None) -> torch.Tensor:
+                        max_count: Optional[int] = None, form: str = "retention") -> torch.Tensor:
     """Retention, token by token: ``proj`` ``[tokens, 2 heads dim + 2 heads vdim]`` holds q, k, v
     and the gate side by side; ``state`` (float32 ``[slots, heads, dim, vdim]``) is read and left
     up to date.  Returns the gated, per-head normalised output ``[tokens, heads * vdim]``.
     ``chunked``: the matrix-core form for bfloat16 prompt portions, 32 tokens at a time (same
     arguments, same state).  With ``max_count`` (the most tokens a row brings) and few rows it
-    takes one workgroup a chunk instead of one a (row, head): what every chunk adds to the state,
-    a scan over the chunks, then every chunk's outputs (:func:`retention_chunk_parallel`)."""
+    takes one workgroup a stretch of chunks instead of one a (row, head): what every stretch adds to the
+    state, a scan over the stretches, then every stretch's outputs (:func:`retention_chunk_parallel`).
+
+    ``form="lightning"``: the same recurrence on ``silu(q)``, ``silu(k)`` and ``silu(v)`` (rounded to the
+    projection's type), no rotation and no scale; the result is float32, neither normed nor gated (the
+    gate's columns are left for :func:`norm_gate`)."""
+    code = RETENTION_FORMS[form]
+    if code and (rot_dims or k_scale != 1.0):
+        raise KernelError("retention: the lightning form neither rotates nor scales")
     if proj.dim() != 2 or proj.shape[1] != 2 * heads * dim + 2 * heads * vdim or proj.stride(1) != 1:
         raise KernelError("retention: the projection's rows must hold q, k, v and the gate")
     tokens = proj.shape[0]
@@ -618,13 +693,14 @@ def retention_recurrent(proj: torch.Tensor, state: torch.Tensor, decay: torch.Te
         raise KernelError("retention: inv_freq must hold rot_dims/2 frequencies")
     if not proj.is_cuda:
         raise KernelError("proj must live on the GPU; there is no CPU path")
-    out = torch.empty((tokens, heads * vdim), dtype=proj.dtype, device=proj.device)
+    out = torch.empty((tokens, heads * vdim), dtype=torch.float32 if code else proj.dtype, device=proj.device)
     if chunked:
         if not retention_chunked_ok(proj.dtype, dim=dim, vdim=vdim, rot_dims=rot_dims):
             raise KernelError("retention: the chunked form does not take this geometry")
-        chunk_state = None
+        chunk_state, span = None, 1
         if max_count is not None and retention_chunk_parallel(rows, heads, dim, vdim, max_count):
-            chunks = -(-max_count // RETENTION_CHUNK)
+            span = retention_chunk_span(rows, heads, max_count)
+            chunks = -(-max_count // (RETENTION_CHUNK * span))
             chunk_state = torch.empty((rows * heads * chunks * dim * vdim,), dtype=torch.float32, device=proj.device)
         _lib.call("pylon_retention_chunked", _dev(out, "out"), proj.data_ptr(), proj.stride(0), 0, heads * dim,
                   2 * heads * dim, 2 * heads * dim + heads * vdim, _dev(state, "state", torch.float32),
@@ -632,14 +708,14 @@ def retention_recurrent(proj: torch.Tensor, state: torch.Tensor, decay: torch.Te
                   _dev(positions, "positions", torch.int32), _dev(row_start, "row_start", torch.int32),
                   _dev(row_slots, "row_slots", torch.int32), rows, heads, dim, vdim, float(eps), float(k_scale),
                   int(max_count or 0), _dev(chunk_state, "chunk_state"),
-                  0 if chunk_state is None else chunk_state.numel(), _stream())
+                  0 if chunk_state is None else chunk_state.numel(), int(span), code, _stream())
         return out
     _lib.call("pylon_retention_recurrent", _dev(out, "out"), proj.data_ptr(), dtype_code(proj.dtype), proj.stride(0),
               0, heads * dim, 2 * heads * dim, 2 * heads * dim + heads * vdim, _dev(state, "state", torch.float32),
               _dev(decay, "decay", torch.float32), _dev(inv_freq, "inv_freq", torch.float32), int(rot_dims),
               _dev(positions, "positions", torch.int32), _dev(row_start, "row_start", torch.int32),
               _dev(row_slots, "row_slots", torch.int32), rows, heads, dim, vdim, float(eps), float(k_scale),
-              _stream())
+              code, _stream())
     return out
 
 
@@ -1228,15 +1304,21 @@ def _streaming_ok(x: torch.Tensor, weight: torch.Tensor, rows: int) -> bool:
             and x.data_ptr() % 16 == 0 and weight.data_ptr() % 16 == 0)
 
 
+def _epilogue(glu: bool, relu2: bool, act: str) -> int:
+    """What the streaming product kernels do to their sums: 0 nothing, 1 and 3 a gate through silu or
+    gelu, 2 the squared relu."""
+    return 2 if relu2 else ((1, 3)[GATE_ACTS[act]] if glu else 0)
+
+
 def gemm_skinny(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype = torch.bfloat16,
                 parts: int = 1, glu: bool = False, relu2: bool = False,
-                out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                out: Optional[torch.Tensor] = None, act: str = "silu") -> torch.Tensor:
     """``x @ weight.T`` for at most 64 rows of bfloat16 ``x``, streaming ``weight`` once.
 
     ``parts > 1`` cuts K into that many ranges and returns float32 partial results
     ``[parts, M, N]`` for the consumer to add.  ``glu``: ``weight`` is a fused
-    ``[2N, K]`` gate/up matrix and the result is ``silu(x @ gate.T) * (x @ up.T)``.  ``relu2``: the
-    result is ``max(x @ weight.T, 0)^2``.
+    ``[2N, K]`` gate/up matrix and the result is ``act(x @ gate.T) * (x @ up.T)`` (:data:`GATE_ACTS`).
+    ``relu2``: the result is ``max(x @ weight.T, 0)^2``.
     """
     if relu2 and (glu or parts > 1):
         raise KernelError("gemm_skinny: the squared relu takes the whole product, and no gate")
@@ -1259,20 +1341,20 @@ def gemm_skinny(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype
             or not out.is_cuda or not out.is_contiguous():
         raise KernelError(f"gemm_skinny: out must be contiguous, on the GPU and of shape {shape}")
     _lib.call("pylon_gemm_skinny", out.data_ptr(), dtype_code(out.dtype), x.data_ptr(), weight.data_ptr(),
-              m, n, k, x.stride(0), weight.stride(0), n, parts, m * n, 2 if relu2 else (1 if glu else 0), _stream())
+              m, n, k, x.stride(0), weight.stride(0), n, parts, m * n, _epilogue(glu, relu2, act), _stream())
     return out
 
 
 def gemm_rows(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype = torch.bfloat16,
               parts: int = 1, col_tiles: int = 1, glu: bool = False, relu2: bool = False, waves: int = 0, cols: int = 0,
-              out: Optional[torch.Tensor] = None) -> torch.Tensor:
+              out: Optional[torch.Tensor] = None, act: str = "silu") -> torch.Tensor:
     """``x @ weight.T`` for at most 128 rows of bfloat16 ``x``: the rows of ``x`` pass through
     LDS once per workgroup of up to 64 (``col_tiles=1``) or 128 (``col_tiles=2``) columns and
     ``weight`` is streamed once (beyond 64 rows each half of the rows has workgroups of its
     own, and two that take the same columns run side by side).  ``parts > 1`` cuts K into that many ranges and returns
     float32 partial results ``[parts, M, N]`` for the consumer to add.  ``glu``: ``weight`` is
-    a fused ``[2N, K]`` gate/up matrix and the result is ``silu(x @ gate.T) * (x @ up.T)``,
-    rounded once.  ``waves``: wavefronts per workgroup, 4 or 2 (0: the kernel's choice);
+    a fused ``[2N, K]`` gate/up matrix and the result is ``act(x @ gate.T) * (x @ up.T)``
+    (:data:`GATE_ACTS`), rounded once.  ``waves``: wavefronts per workgroup, 4 or 2 (0: the kernel's choice);
     ``cols``: columns per workgroup (0: the kernel's choice, an equal share for every
     workgroup of whole rounds over the compute units where that pays).  The sums depend on
     neither.  ``relu2``: the result is ``max(x @ weight.T, 0)^2``, rounded once."""
@@ -1297,7 +1379,7 @@ def gemm_rows(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype =
             or not out.is_cuda or not out.is_contiguous():
         raise KernelError(f"gemm_rows: out must be contiguous, on the GPU and of shape {shape}")
     _lib.call("pylon_gemm_rows", out.data_ptr(), dtype_code(out.dtype), x.data_ptr(), weight.data_ptr(),
-              m, n, k, x.stride(0), weight.stride(0), n, parts, m * n, int(col_tiles), 2 if relu2 else (1 if glu else 0), int(waves),
+              m, n, k, x.stride(0), weight.stride(0), n, parts, m * n, int(col_tiles), _epilogue(glu, relu2, act), int(waves),
               int(cols), _stream())
     return out
 
@@ -1369,8 +1451,8 @@ def linear_for_residual(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: tor
     return linear(x, weight, out_dtype=out_dtype)
 
 
-def linear_glu(x: torch.Tensor, gate_up: torch.Tensor, *, out_dtype: torch.dtype) -> torch.Tensor:
-    """``silu(x @ gate.T) * (x @ up.T)`` for a fused ``[2I, K]`` gate/up matrix.  Up to 128
+def linear_glu(x: torch.Tensor, gate_up: torch.Tensor, *, out_dtype: torch.dtype, act: str = "silu") -> torch.Tensor:
+    """``act(x @ gate.T) * (x @ up.T)`` for a fused ``[2I, K]`` gate/up matrix.  Up to 128
     bfloat16 rows: the activation works on the float32 sums and its result is rounded once
     (in a streaming kernel's epilogue; or, where the library is faster and beyond 64 rows,
     from its float32 result: :func:`plan.plan_gated`).  More rows (prompt portions): the
@@ -1378,11 +1460,11 @@ def linear_glu(x: torch.Tensor, gate_up: torch.Tensor, *, out_dtype: torch.dtype
     if _streaming_ok(x, gate_up, SPLIT_ROWS) and x.is_cuda and gate_up.shape[0] % 2 == 0:
         choice = plan.plan_gated(x.shape[0], gate_up.shape[0] // 2, gate_up.shape[1], gate_up.stride(0))
         if choice.kernel == "rows":
-            return gemm_rows(x, gate_up, out_dtype=out_dtype, glu=True)
+            return gemm_rows(x, gate_up, out_dtype=out_dtype, glu=True, act=act)
         if choice.kernel == "skinny":
-            return gemm_skinny(x, gate_up, out_dtype=out_dtype, glu=True)
-        return silu_gate(_library_float(x, gate_up), out_dtype=out_dtype)
-    return silu_gate(linear(x, gate_up, out_dtype=out_dtype))
+            return gemm_skinny(x, gate_up, out_dtype=out_dtype, glu=True, act=act)
+        return silu_gate(_library_float(x, gate_up), out_dtype=out_dtype, act=act)
+    return silu_gate(linear(x, gate_up, out_dtype=out_dtype), act=act)
 
 
 def linear_relu2(x: torch.Tensor, weight: torch.Tensor, *, out_dtype: torch.dtype) -> torch.Tensor:
@@ -1777,7 +1859,8 @@ def route_top(logits: torch.Tensor, bias: Optional[torch.Tensor], *, n_experts: 
 
 
 def route_scored(logits: torch.Tensor, correction: Optional[torch.Tensor], *, n_experts: int, top: int,
-                 groups: int = 1, keep: int = 1, scale: float = 1.0):
+                 groups: int = 1, keep: int = 1, scale: float = 1.0, scoring: str = "softmax_all",
+                 group_score: str = "max", renormalize: bool = False):
     """From float32 router logits ``[tokens, outputs]``, of which the first ``n_experts`` are experts
     and the others identity experts: scores are the softmax over all outputs; ``correction`` (float32
     ``[outputs]``) is added for the choice only; the outputs form ``groups`` equal groups of
@@ -1785,7 +1868,10 @@ def route_scored(logits: torch.Tensor, correction: Optional[torch.Tensor], *, n_
     the ``top`` largest corrected scores are taken (the lower index among equals).  Returns the
     chosen outputs (int32 ``[tokens, top]``; an identity keeps its index ``>= n_experts``), their
     weights ``score * scale`` (float32 ``[tokens, top]``, zero for an identity) and the sum of the
-    chosen identities' weights (float32 ``[tokens]``; None if every output is an expert)."""
+    chosen identities' weights (float32 ``[tokens]``; None if every output is an expert).
+    ``scoring="sigmoid"``: every output's own sigmoid in place of the softmax.  ``group_score="top2"``: a
+    group counts with the sum of its two largest corrected scores.  ``renormalize``: the weights are
+    ``scale * score / (sum of the chosen scores + 1e-20)``."""
     if logits.dim() != 2 or logits.dtype != torch.float32 or logits.stride(1) != 1:
         raise KernelError("route_scored takes float32 logits [tokens, outputs]")
     tokens, outputs = logits.shape
@@ -1796,7 +1882,8 @@ def route_scored(logits: torch.Tensor, correction: Optional[torch.Tensor], *, n_
     identity = torch.empty((tokens,), dtype=torch.float32, device=logits.device) if outputs > n_experts else None
     _lib.call("pylon_route_scored", _dev(experts, "experts"), _dev(weights, "weights"), _dev(identity, "identity"),
               logits.data_ptr(), logits.stride(0), _dev(correction, "correction", torch.float32), tokens, outputs,
-              n_experts, top, int(groups), int(keep), float(scale), _stream())
+              n_experts, top, int(groups), int(keep), float(scale), {"softmax_all": 0, "sigmoid": 1}[scoring],
+              {"max": 0, "top2": 1}[group_score], 1 if renormalize else 0, _stream())
     return experts, weights, identity
 
 

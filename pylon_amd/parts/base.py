@@ -30,6 +30,8 @@ block         ``forward(resid, delta, ctx, cache, stores) -> (resid, delta)``: t
 stream        ``forward(resid, ctx) -> resid``: the embedded tokens (float32 ``[tokens, dim]``)
               before the first layer: an embedding norm, learned positions
               (``ctx.positions``), a scale.
+pass          ``forward(resid, delta, embedded, t, ctx) -> (resid, delta)``: ahead of pass ``t`` through
+              layers that run several times; ``embedded`` is the stream before the first layer.
 logits        ``forward(logits, ctx) -> logits``: float32 ``[wanted, vocab]`` after the
               vocabulary head: a soft cap, a scale, a bias (in place).
 """
@@ -120,12 +122,13 @@ class Normed:
 @dataclass
 class Scaled:
     """A part's output that is still to get a ``bias`` per element (a projection's bias that was left
-    for the sum), to be multiplied element by element by ``scale`` and added to the residual stream
-    (either may be None).  ``value`` as in :class:`Normed`."""
+    for the sum), to be multiplied element by element by ``scale`` (either may be None) and as a whole by
+    ``factor``, and added to the residual stream.  ``value`` as in :class:`Normed`."""
 
     value: torch.Tensor
     scale: Optional[torch.Tensor] = None
     bias: Optional[torch.Tensor] = None
+    factor: float = 1.0
 
 
 @dataclass
@@ -173,7 +176,8 @@ def summed(delta: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
         value = summed(delta.value)
         if delta.bias is not None:
             value = value + delta.bias.float()
-        return value if delta.scale is None else value * delta.scale.float()
+        value = value if delta.scale is None else value * delta.scale.float()
+        return value if delta.factor == 1.0 else value * delta.factor
     return delta.sum(dim=0) if delta.dim() == 3 else delta.float()
 
 

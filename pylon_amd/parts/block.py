@@ -9,7 +9,8 @@ formed inside the norm kernel that follows it; it hands back the same pair.
 A ``pre_norm`` layer may also have: a short convolution or a token shift on ``norm1``'s output
 (``input_conv``; the norm's output then stays float32 until the shift has rounded it once); a learned
 scale per element on each sublayer's output (``sublayer_scale``); a feed-forward or mixer that leaves
-its output projection's bias to the sum (``output_bias``); and ``depth_mix``: the layer's result is kept
+its output projection's bias to the sum (``output_bias``); one factor on both sublayers' outputs
+(``residual_factor``); and ``depth_mix``: the layer's result is kept
 as one of the streams of the step, and what it hands on is a learned mix of all streams so far.  All of
 these travel to the next norm as :class:`~.base.Scaled` or :class:`~.base.DepthMixed` and cost no launch
 of their own."""
@@ -57,6 +58,8 @@ class PreNormBlock(Part):
             if not 1 <= index < total:
                 raise ValueError(f"a layer's result is stream 1 to {total - 1} of {total}, not {index}")
             self.add_param("depth_coeff", (index + 1,), torch.float32, device, role="vector")
+        if spec.residual_factor != 1.0 and spec.depth_mix is not None:
+            raise ValueError("a layer whose result is mixed with the earlier layers' takes no factor on its sublayers")
         # a sublayer that can leave its last bias to the residual sum is told to
         for part in (self.mixer, self.feed_forward):
             if part is not None and hasattr(part, "defer_output_bias"):
@@ -97,9 +100,9 @@ class PreNormBlock(Part):
         """A sublayer's output with what is still to happen to it on its way into the sum."""
         scale = self.params.get(scale_name)
         bias = getattr(part, "output_bias", None) if getattr(part, "defer_output_bias", False) else None
-        if scale is None and bias is None:
+        if scale is None and bias is None and self.spec.residual_factor == 1.0:
             return value
-        return Scaled(value, scale, bias)
+        return Scaled(value, scale, bias, self.spec.residual_factor)
 
     def _result(self, pending, streams):
         """The layer's last output: as it is, or to be mixed with the earlier layers' results."""
@@ -122,6 +125,8 @@ class SandwichNormBlock(Part):
         super().__init__()
         if spec.mixer_post_norm is None:
             raise ValueError("a sandwich_norm layer needs the norm after its mixer")
+        if spec.residual_factor != 1.0:
+            raise ValueError("a sandwich_norm layer takes no factor on its sublayers")
         if (spec.feed_forward is None) != (spec.feed_forward_norm is None) or \
                 (spec.feed_forward is None) != (spec.feed_forward_post_norm is None):
             raise ValueError("a feed-forward and its two norms come together or not at all")
@@ -170,8 +175,8 @@ class HyperConnectionBlock(PreNormBlock):
     copies, forms the sum that is read next and norms it."""
 
     def __init__(self, spec: LayerSpec, *, dtype: torch.dtype, device) -> None:
-        if spec.input_conv is not None or spec.sublayer_scale or spec.depth_mix is not None:
-            raise ValueError("a layer of hyper-connections has no input convolution, sublayer scales or depth mix")
+        if spec.input_conv is not None or spec.sublayer_scale or spec.depth_mix is not None or spec.residual_factor != 1.0:
+            raise ValueError("a layer of hyper-connections has no input convolution, sublayer scales, factor or depth mix")
         if not 1 <= spec.streams <= ops.STREAM_COPIES:
             raise ValueError(f"hyper-connections take 1 to {ops.STREAM_COPIES} copies of the stream, got {spec.streams}")
         super().__init__(spec, dtype=dtype, device=device)

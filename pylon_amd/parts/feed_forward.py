@@ -14,8 +14,10 @@ from .registry import register_part
 class GatedFeedForward(Part):
     def __init__(self, spec: GatedFeedForwardSpec, *, dtype: torch.dtype, device) -> None:
         super().__init__()
-        if spec.activation != "silu":
-            raise ValueError(f"activation {spec.activation!r} is not supported (only 'silu')")
+        if spec.activation not in ops.GATE_ACTS:
+            raise ValueError(f"activation {spec.activation!r} is not supported (known: {', '.join(ops.GATE_ACTS)})")
+        if spec.bias and spec.activation != "silu":
+            raise ValueError("a gated feed-forward with biases has the activation 'silu'")
         self.spec = spec
         self.dtype = dtype
         element_size = torch.empty((), dtype=dtype).element_size()
@@ -35,7 +37,7 @@ class GatedFeedForward(Part):
 
     def forward(self, h: torch.Tensor, ctx) -> torch.Tensor:
         if not self.spec.bias:
-            hidden = ops.linear_glu(h, self.params["gate_up"], out_dtype=self.dtype)
+            hidden = ops.linear_glu(h, self.params["gate_up"], out_dtype=self.dtype, act=self.spec.activation)
             return ops.linear_for_residual(hidden, self.params["down"], out_dtype=self.dtype)
         sums = ops.linear(h, self.params["gate_up"], out_dtype=torch.float32)
         hidden = ops.gated_act(sums, alpha=1.0, offset=0.0, limit=0.0, out_dtype=self.dtype,

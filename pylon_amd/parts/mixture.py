@@ -20,8 +20,9 @@ only, a choice limited to the best groups of neighbouring outputs, weights that 
 constant, and identity experts (router outputs without matrices, whose output is the input itself:
 the expert kernels pass over them and add the input times the sum of their weights).
 
-``scoring="sigmoid"``: the chosen experts' weights are the sigmoids of their own router outputs, not
-renormalised.  ``weight_on_input``: a chosen expert runs on the token's input times its weight,
+``scoring="sigmoid"``: the chosen experts' weights are the sigmoids of their own router outputs, as they
+are or (``renormalize``) over their sum; with groups a group may count with its largest score or with the
+sum of its two largest.  ``weight_on_input``: a chosen expert runs on the token's input times its weight,
 ``sum_e expert_e(w_e h)``; the token-by-token kernel scales the input in float32 as it stages it, the
 sorted path scales the gate's and the up's float32 sums before the activation (the same number,
 because the two products are linear).
@@ -53,17 +54,26 @@ class MixtureFeedForward(Part):
         if spec.weight_on_input and (spec.expert_act != "silu_gated" or spec.n_identity):
             raise ValueError("weights on the experts' inputs go with gated experts and without identity experts")
         outputs = spec.n_experts + spec.n_identity
-        if spec.scoring in ("top_softmax", "sigmoid"):
-            if spec.n_identity or spec.groups != 1 or spec.route_scale != 1.0:
-                raise ValueError("identity experts, groups and a scale of the weights belong to the scoring softmax_all")
+        if spec.group_score not in ("max", "top2"):
+            raise ValueError(f"unknown score of a group {spec.group_score!r} (known: max, top2)")
+        # the plain ways to choose have a kernel of their own; groups and weights over their sum go with
+        # the scored one
+        self.scored = spec.scoring == "softmax_all" or (spec.scoring == "sigmoid" and (spec.groups != 1 or spec.renormalize))
+        if spec.scoring != "softmax_all" and (spec.n_identity or spec.route_scale != 1.0):
+            raise ValueError("identity experts and a scale of the weights belong to the scoring softmax_all")
+        if not self.scored:
+            if spec.groups != 1 or spec.renormalize:
+                raise ValueError("groups and weights over their sum belong to the scorings softmax_all and sigmoid")
         else:
             if spec.n_identity < 0 or outputs > 512 or spec.top > outputs:
                 raise ValueError(f"the router has 1 to 512 outputs and a token takes at most all of them, not {spec.top} of {outputs}")
             if spec.groups < 1 or outputs % spec.groups or not 1 <= spec.groups_kept <= spec.groups:
                 raise ValueError(f"{outputs} router outputs do not form {spec.groups} equal groups of which "
                                  f"{spec.groups_kept} are kept")
+            if spec.scoring == "sigmoid" and spec.top > outputs // spec.groups * spec.groups_kept:
+                raise ValueError(f"{spec.groups_kept} groups of {outputs // spec.groups} outputs do not hold {spec.top} choices")
             if spec.shared_gate:
-                raise ValueError("the gate of a shared expert is one more router row of the scoring top_softmax only")
+                raise ValueError("the gate of a shared expert is one more router row of the plain ways to choose only")
         self.spec = spec
         self.dtype = dtype
         self.gated = spec.expert_act == "silu_gated"
@@ -91,11 +101,12 @@ class MixtureFeedForward(Part):
         spec = self.spec
         logits = ops.linear(h, self.params["router"], out_dtype=torch.float32)
         identity = None
-        if spec.scoring == "softmax_all":
+        if self.scored:
             shared_gate = None
             experts, weights, identity = ops.route_scored(
                 logits, self.params.get("router_bias"), n_experts=spec.n_experts, top=spec.top, groups=spec.groups,
-                keep=spec.groups_kept, scale=spec.route_scale)
+                keep=spec.groups_kept, scale=spec.route_scale, scoring=spec.scoring, group_score=spec.group_score,
+                renormalize=spec.renormalize)
         else:
             experts, weights, shared_gate = ops.route_top(
                 logits, self.params.get("router_bias"), n_experts=spec.n_experts, top=spec.top,

@@ -53,9 +53,13 @@ class RMSNorm(Part):
                                 out_dtype=self.dtype)
             return out if fused else ops.rmsnorm(resid, self.weight(), self.spec.eps, out_dtype=self.dtype,
                                                  row_idx=row_idx)
+        if isinstance(delta, Scaled) and delta.scale is None and delta.bias is None:
+            return ops.add_rmsnorm(resid, delta.value, self.weight(), self.spec.eps, self.dtype, row_idx=row_idx,
+                                   factor=delta.factor)
         if isinstance(delta, Scaled):
             return ops.add_normed_rmsnorm(resid, delta.value, self.weight(), self.spec.eps, self.dtype,
-                                          row_idx=row_idx, delta_scale=delta.scale, delta_bias=delta.bias)
+                                          row_idx=row_idx, delta_scale=delta.scale, delta_bias=delta.bias,
+                                          factor=delta.factor)
         return ops.add_rmsnorm(resid, delta, self.weight(), self.spec.eps, self.dtype,
                                row_idx=row_idx)
 
@@ -121,6 +125,10 @@ class ScalarRMSNorm(Part):
         if isinstance(delta, Normed):
             return ops.add_normed_rmsnorm(resid, delta.value, self.params["weight"], self.spec.eps, self.dtype,
                                           post_gain=delta.gain, post_eps=delta.eps, row_idx=row_idx)
+        if isinstance(delta, Scaled) and not isinstance(delta, DepthMixed):
+            return ops.add_normed_rmsnorm(resid, delta.value, self.params["weight"], self.spec.eps, self.dtype,
+                                          row_idx=row_idx, delta_scale=delta.scale, delta_bias=delta.bias,
+                                          factor=delta.factor)
         return ops.add_normed_rmsnorm(resid, delta, self.params["weight"], self.spec.eps, self.dtype, row_idx=row_idx)
 
 

@@ -14,7 +14,7 @@ from typing import Optional, Tuple
 
 import torch
 
-from ..config.specs import PositionSpec, SinusoidPositionSpec
+from ..config.specs import PositionSpec, RotaryBandScalingSpec, SinusoidPositionSpec
 from ..kernels import ops
 from .base import Part
 from .registry import register_part
@@ -28,7 +28,9 @@ class RotaryPosition(Part):
         self.spec = spec
         self.interleaved = spec.interleaved
         self.rot_scale = 1.0  # what every cosine and sine is multiplied by
-        if spec.scaling is not None:
+        if isinstance(spec.scaling, RotaryBandScalingSpec):
+            inv_freq = band_frequencies(spec)
+        elif spec.scaling is not None:
             inv_freq, self.rot_scale = scaled_frequencies(spec)
         elif spec.interleaved:
             # neighbours (2i, 2i + 1) turn together; frequencies theta ** (-2i/d) formed in double
@@ -64,6 +66,28 @@ def scaled_frequencies(spec: PositionSpec):
     ramp = ((index - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
     freq = plain / sc.factor * ramp + plain * (1.0 - ramp)
     return freq.to(torch.float32), 0.1 * math.log(sc.factor) + 1.0
+
+
+def band_frequencies(spec: PositionSpec) -> torch.Tensor:
+    """float32 frequencies of the rotary_dim / 2 pairs of a rotation whose slow pairs are stretched by
+    wavelength (:class:`RotaryBandScalingSpec`); formed in double precision and rounded once."""
+    import math
+
+    sc, dims = spec.scaling, spec.rotary_dim
+    if not (sc.factor > 0 and sc.original > 0 and 0 < sc.low < sc.high):
+        raise ValueError("a rotation scaled by wavelength needs a positive factor and original and 0 < low < high")
+    out = []
+    for i in range(dims // 2):
+        f = float(spec.theta) ** (-2.0 * i / dims)
+        turns = sc.original * f / (2.0 * math.pi)  # over the original length
+        if turns > sc.high:
+            out.append(f)
+        elif turns < sc.low:
+            out.append(f / sc.factor)
+        else:
+            s = (turns - sc.low) / (sc.high - sc.low)
+            out.append((1.0 - s) * f / sc.factor + s * f)
+    return torch.tensor(out, dtype=torch.float64).to(torch.float32)
 
 
 class NoPosition(Part):

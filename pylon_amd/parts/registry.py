@@ -5,13 +5,14 @@ mixer, feed-forward, norm, position encoding or block arrangement is added by
 registering a class; no file of the framework has to change.  Two more families hold what
 a model may do outside its layers: "stream" parts work on the embedded tokens before the
 first layer, "logits" parts on the logits after the vocabulary head.  "conv" parts are short
-convolutions over time that a block may put in front of a sublayer.
+convolutions over time that a block may put in front of a sublayer; a "pass" part changes the stream
+ahead of every pass through layers that run several times.
 """
 from __future__ import annotations
 
 from typing import Callable, Dict
 
-_FAMILIES = ("mixer", "feed_forward", "norm", "position", "block", "stream", "logits", "conv")
+_FAMILIES = ("mixer", "feed_forward", "norm", "position", "block", "stream", "logits", "conv", "pass")
 _PARTS: Dict[str, Dict[str, Callable]] = {family: {} for family in _FAMILIES}
 
 
