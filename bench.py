@@ -2,7 +2,7 @@
 and uniform-random token ids, on one MI355X.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--layers L]
-                    [--shape 4b|8b|32b] [--prompt-len N] [--design vupuzen|pavitar|gimudra|tukarax|ranudra [--beside qwen3|vupuzen|pavitar|gimudra] [--design-shapes 8b,...]]
+                    [--shape 4b|8b|32b] [--prompt-len N] [--design vupuzen|pavitar|gimudra|tukarax|ranudra|farorax [--beside qwen3|vupuzen|pavitar|gimudra|tukarax|ranudra] [--design-shapes 8b,...]]
 
 Everything goes the product's own way.  Start-up is ``Runner.from_random``: the fit check,
 the measured activation headroom, the page pool sized from the card's memory and the decode
@@ -405,6 +405,36 @@ def ranudra_json(shape: dict, layers: int) -> dict:
             "layers": [(linear, first, second)[i % 3] for i in range(own)]}
 
 
+def farorax_json(shape: dict, layers: int) -> dict:
+    """A Farorax configuration of the shape's layer sizes: of every four layers two lightning attention
+    (as many heads of the shape's head size as fill half the width) and two attention (the shape's heads,
+    rotated whole, windows of 1,024 positions); of each kind one has the shape's feed-forward and the other
+    a mixture of 32 experts in 4 groups of which 2 are kept, 4 a token, with a shared expert, sized so that
+    a token's experts together are about as large as the feed-forward; the shape's vocabulary.  Of ``layers``
+    runs the middle stretch runs twice over the same weights (a quarter fewer layers own weights)."""
+    width, hd = shape["hidden_size"], shape["head_dim"]
+    expert = max(64, shape["intermediate_size"] // 6 // 64 * 64)
+    dense = {"kind": "dense", "ff": shape["intermediate_size"]}
+    moe = {"kind": "moe", "expert": {"ff": expert}, "shared": {"ff": 2 * expert},
+           "router": {"experts": 32, "top": 4, "groups": {"count": 4, "keep": 2}}}
+    heads = max(1, width // (2 * hd))
+    decay = [1.0 - 2.0 ** (-1 - 8 * h / max(1, heads - 1)) for h in range(heads)]
+    lightning = {"heads": heads, "dim": hd, "vdim": hd, "decay": decay}
+    attention = {"heads": shape["num_attention_heads"], "kv_heads": shape["num_key_value_heads"], "dim": hd, "vdim": hd,
+                 "scale": hd ** -0.5, "mask": {"size": 1024},
+                 "rot": {"base": 500000.0, "dims": hd,
+                         "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    kinds = [{"type": "lightning", "mixer": lightning, "mlp": dense}, {"type": "attention", "mixer": attention, "mlp": moe},
+             {"type": "lightning", "mixer": lightning, "mlp": moe}, {"type": "attention", "mixer": attention, "mlp": dense}]
+    again = layers // 4  # this many layers run twice
+    own = layers - again
+    start = (own - again) // 2
+    return {"architecture": "Farorax", "vocab": shape["vocab_size"], "width": width, "norm": {"eps": 1e-6},
+            "residual_mult": 0.25, "logit_softcap": 40.0,
+            "loop": {"start": start, "stop": start + again, "times": 2} if again else None,
+            "layers": [kinds[i % 4] for i in range(own)]}
+
+
 def design_steps(runner, vocab: int, batch: int, prompt_len: int, steps: int, warmup: int, seed: int) -> dict:
     """Milliseconds of one prompt step of ``prompt_len`` tokens (median of five), and of a
     decode step of ``batch`` requests behind such prompts (mean of ``steps``), through the step
@@ -446,7 +476,7 @@ def design_steps(runner, vocab: int, batch: int, prompt_len: int, steps: int, wa
 
 
 def design_main(args) -> int:
-    """``--design vupuzen|pavitar|gimudra|tukarax|ranudra``: prefill and decode of models of that design of random
+    """``--design vupuzen|pavitar|gimudra|tukarax|ranudra|farorax``: prefill and decode of models of that design of random
     weights at the layer sizes of ``--shape`` (and of the other shapes named by ``--design-shapes``),
     beside the model of the design ``--beside`` (Qwen3 unless told otherwise) of the same sizes and
     number of layer runs, both through the same step function over pages of 256 tokens with decode
@@ -468,7 +498,7 @@ def design_main(args) -> int:
         layers = args.layers or 8
         pages = (args.batch + 1) * (-(-(prompt_len + steps + warmup + 8) // PAGE_SIZE) + 1)
         makers = {"vupuzen": vupuzen_json, "pavitar": pavitar_json, "gimudra": gimudra_json, "tukarax": tukarax_json,
-                  "ranudra": ranudra_json, "qwen3": config_json}
+                  "ranudra": ranudra_json, "farorax": farorax_json, "qwen3": config_json}
         for design, raw in ((args.design, makers[args.design](shape, layers)), (beside, makers[beside](shape, layers))):
             config = PylonConfig(dtype=args.dtype, max_batch_size=args.batch + 1, max_queue_size=args.batch + 1,
                                  page_size=PAGE_SIZE, prefill_chunk_size=prompt_len, num_pages=pages,
@@ -519,9 +549,9 @@ def main() -> int:
     parser.add_argument("--no-peaks", action="store_true", help="skip the probes of this device's own peaks")
     parser.add_argument("--mixed", action="store_true",
                         help="also time a step of --batch decoded tokens beside a 2,048-token prompt portion")
-    parser.add_argument("--design", choices=("qwen3", "vupuzen", "pavitar", "gimudra", "tukarax", "ranudra"), default="qwen3",
-                        help="vupuzen, pavitar, gimudra, tukarax, ranudra: that design beside Qwen3 at equal sizes instead of the default workload")
-    parser.add_argument("--beside", choices=("qwen3", "vupuzen", "pavitar", "gimudra", "tukarax"), default="qwen3",
+    parser.add_argument("--design", choices=("qwen3", "vupuzen", "pavitar", "gimudra", "tukarax", "ranudra", "farorax"), default="qwen3",
+                        help="vupuzen, pavitar, gimudra, tukarax, ranudra, farorax: that design beside Qwen3 at equal sizes instead of the default workload")
+    parser.add_argument("--beside", choices=("qwen3", "vupuzen", "pavitar", "gimudra", "tukarax", "ranudra"), default="qwen3",
                         help="with another --design: the design it is measured beside (default qwen3)")
     parser.add_argument("--design-shapes", default="", help="with another --design: further shapes, with commas")
     parser.add_argument("--prefill-only", action="store_true",

@@ -50,6 +50,11 @@ __device__ __forceinline__ bf16_t from_float<bf16_t>(float v) {
 #define PYLON_ACT_SILU 0
 #define PYLON_ACT_GELU 1
 __device__ __forceinline__ float pylon_silu(float z) { return z / (1.0f + expf(-z)); }
+// For results that are about to be rounded to bfloat16: the hardware's exponential and reciprocal (about one
+// part in 2^22 each).
+__device__ __forceinline__ float pylon_silu_for_bf16(float z) {
+  return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
 __device__ __forceinline__ float pylon_gelu_tanh(float z) {
   return z / (1.0f + expf(-1.5957691216057308f * fmaf(0.044715f * z * z, z, z)));
 }

@@ -15,7 +15,8 @@ __global__ __launch_bounds__(256) void pass_join_kernel(TO* __restrict__ out, co
   const size_t row = blockIdx.x;
   TO* yr = out + row * 2 * dim;
   const TD* dr = delta ? delta + row * dim : nullptr;
-  for (int i = threadIdx.x; i < dim; i += blockDim.x) {
+  const int i = blockIdx.y * 256 + threadIdx.x;
+  if (i < dim) {
     float v = resid[row * dim + i];
     if (dr) {
       float d = to_float(dr[i]);
@@ -37,7 +38,7 @@ extern "C" int pylon_pass_join(void* out, int out_dtype, const float* resid, con
   PYLON_REQUIRE(rows >= 0 && dim > 0 && n_delta >= 1, "pass_join: bad sizes");
   if (rows == 0) return 0;
 #define GO(TD, TO)                                                                                                \
-  hipLaunchKernelGGL((pass_join_kernel<TD, TO>), dim3(rows), dim3(256), 0, stream, (TO*)out, resid, (const TD*)delta, \
+  hipLaunchKernelGGL((pass_join_kernel<TD, TO>), dim3(rows, (dim + 255) / 256), dim3(256), 0, stream, (TO*)out, resid, (const TD*)delta, \
                      n_delta, delta_stride, factor, embedded, dim)
   if (delta_dtype == PYLON_F32 && out_dtype == PYLON_F32) GO(float, float);
   else if (delta_dtype == PYLON_F32) GO(float, bf16_t);
@@ -51,7 +52,8 @@ __global__ __launch_bounds__(256) void pass_begin_kernel(float* __restrict__ res
                                                          int n_parts, long long part_stride,
                                                          const float* __restrict__ step, int dim) {
   const size_t row = blockIdx.x;
-  for (int i = threadIdx.x; i < dim; i += blockDim.x) {
+  const int i = blockIdx.y * 256 + threadIdx.x;
+  if (i < dim) {
     float v = product[row * dim + i];
 #pragma unroll 4
     for (int p = 1; p < n_parts; ++p) v += product[row * dim + i + p * part_stride];
@@ -65,6 +67,7 @@ extern "C" int pylon_pass_begin(float* resid, const float* product, int n_parts,
                                 const float* step, int rows, int dim, hipStream_t stream) {
   PYLON_REQUIRE(rows >= 0 && dim > 0 && n_parts >= 1, "pass_begin: bad sizes");
   if (rows == 0) return 0;
-  hipLaunchKernelGGL(pass_begin_kernel, dim3(rows), dim3(256), 0, stream, resid, product, n_parts, part_stride, step, dim);
+  hipLaunchKernelGGL(pass_begin_kernel, dim3(rows, (dim + 255) / 256), dim3(256), 0, stream, resid, product, n_parts,
+                     part_stride, step, dim);
   PYLON_LAUNCHED("pass_begin");
 }

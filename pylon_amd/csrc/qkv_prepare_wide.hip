@@ -120,6 +120,70 @@ qkv_prepare_wide_kernel(T* __restrict__ q_out, T* __restrict__ k_cache, T* __res
   }
 }
 
+// The same without norms, for neighbours that turn together, sixteen bytes (four pairs) at a time: bfloat16,
+// head sizes, rotated part, row stride and offsets multiples of 8 elements.  blockIdx.x is a token, blockIdx.y
+// a share of its pieces (few tokens: several workgroups each).  With `fold` the workgroups of one die take
+// neighbouring tokens (workgroups go round the eight dies), so that values written transposed, two bytes a
+// token in a line, meet in that die's cache.
+__global__ void __launch_bounds__(QW_THREADS)
+qkv_rotate_pieces_kernel(bf16_t* __restrict__ q_out, bf16_t* __restrict__ k_cache, bf16_t* __restrict__ v_cache,
+                         const bf16_t* __restrict__ qkv, long long row_stride, const float* __restrict__ inv_freq,
+                         int rot_dim, const int* __restrict__ positions, const int* __restrict__ slot_map, int q_size,
+                         int k_size, int v_size, int head_dim, int store, float rot_scale, int v_offset, int v_page,
+                         int fold) {
+  extern __shared__ float turn[];  // cos then sin of the token's rot_dim/2 angles
+  const int share = fold > 0 ? static_cast<int>(gridDim.x) / 8 : 0;
+  const int b = blockIdx.x;
+  const int t = share > 0 && b < share * 8 ? (b & 7) * share + (b >> 3) : b;
+  const int tid = threadIdx.x, half = rot_dim / 2;
+  const bf16_t* row = qkv + static_cast<size_t>(t) * row_stride;
+  const float pos = rot_dim > 0 ? static_cast<float>(positions[t]) : 0.f;
+  for (int i = tid; i < half; i += QW_THREADS) {
+    float s, c;
+    sincosf(pos * inv_freq[i], &s, &c);
+    turn[i] = c * rot_scale;
+    turn[half + i] = s * rot_scale;
+  }
+  __syncthreads();
+  const int slot = store ? slot_map[t] : 0;
+  const int qp = q_size / 8, kp = store ? k_size / 8 : 0, vp = store ? v_size / 8 : 0;
+  for (int p = blockIdx.y * QW_THREADS + tid; p < qp + kp + vp; p += gridDim.y * QW_THREADS) {
+    if (p < qp + kp) {
+      const int e = (p < qp ? p : p - qp) * 8, d = e % head_dim;
+      const uint4 raw = *reinterpret_cast<const uint4*>(row + (p < qp ? 0 : q_size) + e);
+      uint4 y = raw;
+      if (d < rot_dim) {
+        const uint32_t in[4] = {raw.x, raw.y, raw.z, raw.w};
+        uint32_t o[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float u = __uint_as_float(in[j] << 16), v = __uint_as_float(in[j] & 0xffff0000u);
+          const float c = turn[(d >> 1) + j], s = turn[half + (d >> 1) + j];
+          o[j] = static_cast<uint32_t>(float_to_bf16_bits(u * c - v * s)) |
+                 (static_cast<uint32_t>(float_to_bf16_bits(v * c + u * s)) << 16);
+        }
+        y = uint4{o[0], o[1], o[2], o[3]};
+      }
+      bf16_t* dst = p < qp ? q_out + static_cast<size_t>(t) * q_size : k_cache + static_cast<size_t>(slot) * k_size;
+      *reinterpret_cast<uint4*>(dst + e) = y;
+    } else {
+      const int e = (p - qp - kp) * 8;
+      const uint4 raw = *reinterpret_cast<const uint4*>(row + v_offset + e);
+      if (v_page > 0) {
+        uint16_t* dst = reinterpret_cast<uint16_t*>(v_cache) + (static_cast<size_t>(slot / v_page) * v_size + e) * v_page + slot % v_page;
+        const uint32_t in[4] = {raw.x, raw.y, raw.z, raw.w};
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          dst[static_cast<size_t>(2 * j) * v_page] = static_cast<uint16_t>(in[j] & 0xffffu);
+          dst[static_cast<size_t>(2 * j + 1) * v_page] = static_cast<uint16_t>(in[j] >> 16);
+        }
+      } else {
+        *reinterpret_cast<uint4*>(v_cache + static_cast<size_t>(slot) * v_size + e) = raw;
+      }
+    }
+  }
+}
+
 // qkv: [tokens, n_heads*head_dim (+ n_kv_heads*head_dim + n_kv_heads*v_dim with store)], rows
 // row_stride elements apart.  q_out: [tokens, n_heads, head_dim].  k_cache: [slots, n_kv_heads,
 // head_dim], v_cache: [slots, n_kv_heads, v_dim], slot_map[t] the token's slot.  q_weight
@@ -154,6 +218,20 @@ extern "C" int pylon_qkv_prepare_wide(void* q_out, void* k_cache, void* v_cache,
   if (tokens == 0) return 0;
   const size_t lds = sizeof(float) * ((rot_dim > 0 ? rot_dim : 1) + n_heads + n_kv_heads);
   PYLON_REQUIRE(lds <= 60 * 1024, "qkv_prepare_wide: too many heads");
+  const uintptr_t ends = reinterpret_cast<uintptr_t>(q_out) | reinterpret_cast<uintptr_t>(k_cache) |
+                         reinterpret_cast<uintptr_t>(v_cache) | reinterpret_cast<uintptr_t>(qkv);
+  if (dtype == PYLON_BF16 && q_weight == nullptr && k_weight == nullptr && (rot_dim == 0 || interleaved) &&
+      head_dim % 8 == 0 && rot_dim % 8 == 0 && v_dim % 8 == 0 && v_offset % 8 == 0 && row_stride % 8 == 0 &&
+      (ends & 15) == 0) {
+    const int q_size = n_heads * head_dim, k_size = n_kv_heads * head_dim, v_size = n_kv_heads * v_dim;
+    const int pieces = (q_size + (store ? k_size + v_size : 0)) / 8;
+    const int shares = tokens <= 256 ? (pieces + QW_THREADS - 1) / QW_THREADS : 1;
+    hipLaunchKernelGGL(qkv_rotate_pieces_kernel, dim3(tokens, shares), dim3(QW_THREADS), lds, stream, (bf16_t*)q_out,
+                       (bf16_t*)k_cache, (bf16_t*)v_cache, (const bf16_t*)qkv, row_stride, inv_freq, rot_dim, positions,
+                       slot_map, q_size, k_size, v_size, head_dim, store, rot_scale, v_offset, v_page,
+                       shares == 1 ? 1 : 0);
+    PYLON_LAUNCHED("qkv_prepare_wide");
+  }
   if (dtype == PYLON_F32)
     hipLaunchKernelGGL((qkv_prepare_wide_kernel<float>), dim3(tokens), dim3(QW_THREADS), lds, stream, (float*)q_out,
                        (float*)k_cache, (float*)v_cache, (const float*)qkv, row_stride, q_weight, k_weight, eps,

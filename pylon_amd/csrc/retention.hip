@@ -52,7 +52,7 @@ __global__ __launch_bounds__(THREADS) void retention_recurrent_kernel(void* __re
       const T* src = pr + (is_k ? k_off : q_off) + head * dim;
       float v = to_float(src[d]);
       if (FORM == 1) {
-        v = to_float(from_float<T>(pylon_silu(v)));
+        v = sizeof(T) == 2 ? to_float(from_float<T>(pylon_silu_for_bf16(v))) : pylon_silu(v);
       } else if (d < rot_dims) {
         const int pair = d < half ? d : d - half;
         const float angle = pos * inv_freq[pair];
@@ -66,7 +66,7 @@ __global__ __launch_bounds__(THREADS) void retention_recurrent_kernel(void* __re
     }
     __syncthreads();
     float vj = to_float(pr[v_off + head * vdim + j]);
-    if (FORM == 1) vj = to_float(from_float<T>(pylon_silu(vj)));
+    if (FORM == 1) vj = sizeof(T) == 2 ? to_float(from_float<T>(pylon_silu_for_bf16(vj))) : pylon_silu(vj);
     float acc = 0.f;
     if (owner) {
 #pragma unroll

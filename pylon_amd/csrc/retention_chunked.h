@@ -44,14 +44,15 @@ __device__ __forceinline__ void rc_split1(float a, uint16_t& hi, uint16_t& lo) {
   lo = static_cast<uint16_t>(__float_as_uint(a - __uint_as_float(ua & 0xffff0000u)) >> 16);
 }
 
-// silu of a bfloat16 number, rounded to bfloat16; the recurrent form computes it the same way.
-__device__ __forceinline__ uint16_t rc_silu(uint16_t bits) {
-  return float_to_bf16_bits(pylon_silu(bf16_bits_to_float(bits)));
-}
+// silu of bfloat16 numbers, rounded to bfloat16; the recurrent form computes it the same way.
+typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
+typedef float floatx2 __attribute__((ext_vector_type(2)));
 __device__ __forceinline__ uint32_t rc_silu2(uint32_t pair) {
-  return static_cast<uint32_t>(rc_silu(static_cast<uint16_t>(pair & 0xffffu))) |
-         (static_cast<uint32_t>(rc_silu(static_cast<uint16_t>(pair >> 16))) << 16);
+  const floatx2 y = {pylon_silu_for_bf16(__uint_as_float(pair << 16)),
+                     pylon_silu_for_bf16(__uint_as_float(pair & 0xffff0000u))};
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(y, bf16x2));
 }
+__device__ __forceinline__ uint16_t rc_silu(uint16_t bits) { return static_cast<uint16_t>(rc_silu2(bits)); }
 
 #define RC_MFMA(a, b, c) __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), c, 0, 0, 0)
 

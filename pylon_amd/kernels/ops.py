@@ -647,12 +647,18 @@ def retention_chunk_parallel(rows: int, heads: int, dim: int, vdim: int, max_cou
 
 
 def retention_chunk_span(rows: int, heads: int, max_count: int, units: Optional[int] = None) -> int:
-    """Chunks of 32 tokens a workgroup of the chunk-parallel form walks: as many as still leave two
-    workgroups for every compute unit (a stretch's state is written, scanned and read once, so longer
-    stretches move fewer bytes)."""
+    """Chunks of 32 tokens a workgroup of the chunk-parallel form walks: as few as leave at most one
+    workgroup for every compute unit, or two or three where that would take more than six chunks a workgroup
+    (a stretch's state is written, scanned and read once, so longer stretches move fewer bytes; a number of
+    workgroups just above a multiple of the units leaves the last round almost empty)."""
     units = units or _lib.compute_units()
     chunks = -(-max_count // RETENTION_CHUNK)
-    return max(1, rows * heads * chunks // (2 * units))
+    for rounds in (1, 2, 3):
+        fit = rounds * units // (rows * heads)  # stretches a (row, head) may have
+        span = -(-chunks // fit) if fit else chunks
+        if span <= 6:
+            break
+    return span
 
 
 def retention_chunked_ok(dtype: torch.dtype, *, dim: int, vdim: int, rot_dims: int) -> bool:
